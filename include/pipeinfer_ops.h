@@ -366,6 +366,50 @@ PI_API int pi_op_moe_experts_grouped_glu(const pi_weight * w_up, const pi_weight
  * pi_op_glu_mul); gate_col >= 0: one more column of the same rows holds a per-token gate */
 PI_API int pi_op_glu_mul_ex(const float * in_dev, int64_t in_stride, int ff, int glu, float limit, int64_t gate_col, int n_tok, float * out_dev, int64_t out_stride, void * stream);
 
+/* ---- operators of blocks over several residual streams, of normalised matrix memories, of latent attention with a rotated part and a window, and of query temperatures ------------ */
+/* pi_op_dense with a bias per row (nullable, fp32 [rows]) added ahead of the activation */
+PI_API int pi_op_dense_bias(const pi_weight * w, const float * bias_dev, const float * x_dev, int64_t x_stride, int n_tok, float * out_dev, int64_t out_stride, int act_a, int64_t rows_a, int act_b, int exact, void * stream);
+/* One step of a residual made of `streams` copies x_s per token, and the norm of what the next sublayer reads, in one launch (R(u) = u / sqrt(mean(u^2) + eps)):
+ *   x_t <- sum_s mix[s][t] x_s + out[t] * y   (all from the old ones; mix nullable: x_t stays; y nullable)  -> x_out [n_tok][streams][n] (nullable: not stored; may be x_in when the strides are those of x_out)
+ *   h = R(sum_s in_next[s] x_s) * w           (in_next nullable: the plain sum)
+ * x_in: stream s of token t at x_in + t * token_stride + s * stream_stride (stream_stride 0: every stream is the same row).  At most PI_MAX_STREAMS streams, rows of at most 16384 values */
+#define PI_MAX_STREAMS 16
+PI_API int pi_op_hyper_step(const float * x_in_dev, int64_t token_stride, int64_t stream_stride, int streams, const float * y_dev, int64_t y_stride, const float * mix_dev, const float * out_dev, const float * in_next_dev,
+                            const float * w_dev, float eps, int n, int n_tok, float * x_out_dev, float * h_out_dev, int64_t h_stride, void * stream);
+/* the gates of a normalised matrix memory, fp32:  i = cap tanh((raw_i + bias_i) / cap),  f = log sigmoid(cap tanh((raw_f + bias_f) / cap)),  m' = max(f + m, i)  per head and token, m from
+ * m_state_dev [slots][heads] (0 for a sequence that starts) and back into it;  forget = e^(f + m - m'), put = e^(i - m'), floor = e^(-m'), each [n_tok][heads].  rec_dev as for pi_op_linear_attention */
+PI_API int pi_op_memory_gates(const float * raw_i_dev, const float * raw_f_dev, int64_t stride, const float * bias_i_dev, const float * bias_f_dev, float cap, int heads, float * m_state_dev, const int32_t * rec_dev, int n_tok,
+                              float * forget_dev, float * put_dev, float * floor_dev, void * stream);
+/* pi_op_linear_attention_ex over value_cols value columns and, with key_sum != 0, one more column whose values are 1: its state is the decayed sum of the keys, its output that sum's product with the
+ * query.  State and output rows then have value_cols + 1 columns per head (pi_op_linear_attention_scratch_floats with that many) */
+PI_API int pi_op_linear_attention_keysum(const float * q_dev, const float * k_dev, const float * v_dev, int64_t stride, int heads, int qk_heads, int dim, int value_cols, int key_sum, const float * decay_dev, const float * tdecay_dev,
+                                         const float * tscale_dev, int64_t t_stride, const float * skip_dev, float * state_dev, const int32_t * rec_dev, int n_tok, int max_segments, float * scratch_dev,
+                                         size_t scratch_floats, float * out_dev, int64_t out_stride, void * stream);
+/* what a normalised memory hands on: o = q_mult * y[h][0 .. vdim) / (max(|q_mult * y[h][vdim]|, floor[t][h]) + add) per head (rows of pi_op_linear_attention_keysum), then
+ * o / sqrt(mean(o^2) + eps) * w[h * vdim ..] * act(gate) (gate_act PI_ACT_NONE, _SIGMOID or _SILU; gate nullable) */
+PI_API int pi_op_memory_norm(const float * y_dev, int64_t y_stride, const float * floor_dev, float q_mult, float add, int heads, int vdim, float eps, const float * w_dev, const float * gate_dev, int64_t gate_stride, int gate_act,
+                             int n_tok, float * out_dev, int64_t out_stride, void * stream);
+/* pi_rotary_table_create with angle steps stretched along a ramp over the pair index: with j(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(j(fast)), 0), hi = min(ceil(j(slow)), dims - 1) and
+ * r = clamp((i - lo) / max(hi - lo, 0.001), 0, 1) the step f_i becomes f_i / factor * r + f_i * (1 - r); cos and sin are multiplied by 0.1 ln(factor) + 1 */
+PI_API void * pi_rotary_table_create_ramp(int n_pos, int dims, float base, float factor, int original, float fast, float slow);
+/* pi_op_qkv_prepare_ex with a query temperature, q *= 1 + temp_coef * ln(floor((pos + 1) / temp_every) + 1) behind norm and rotation (temp_every 0: none); k_dev and v_dev NULL: the queries alone (a layer
+ * that reads another layer's cache) */
+PI_API int pi_op_qkv_prepare_temp(const float * q_dev, const float * k_dev, const float * v_dev, int64_t stride, const float * q_norm_w, const float * k_norm_w, float eps, int heads, int kv_heads, int dim, int vdim,
+                                  const void * rotary_table, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every, const int32_t * pos_dev, int n_tok, float * q_out_dev, int64_t q_out_stride,
+                                  float * k_cache_dev, float * v_cache_dev, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream);
+/* the mask rows of a sliding window: out[t] = the bits of mask[t] whose cells hold positions above pos[t] - size.  The cells of the pass learn their positions first (cell_pos_dev) */
+PI_API int pi_op_window_mask(const uint32_t * mask_dev, const int32_t * pos_dev, int32_t * cell_pos_dev, int size, int n_tok, int n_kv, uint32_t * out_mask_dev, const int32_t * dyn_dev, void * stream);
+/* the two latents of a latent attention whose queries go through one as well.  A row of p is [query latent (q_rank) | key / value latent (kv_rank) | rotated key part (rot_dim) | ..]: the query latent
+ * RMS-normed * q_norm_w -> q_latent_dev; the other one RMS-normed * kv_norm_w and, behind it, the key part turned in neighbouring pairs by the token's position -> the token's row of cache_dev [cells][kv_rank + rot_dim] */
+PI_API int pi_op_latent_prepare(const float * p_dev, int64_t p_stride, int q_rank, const float * q_norm_w, int kv_rank, const float * kv_norm_w, int rot_dim, const void * rotary_table, float eps, const int32_t * pos_dev, int n_tok,
+                                float * q_latent_dev, int64_t q_latent_stride, float * cache_dev, const int32_t * dyn_dev, void * stream);
+/* pi_op_latent_attention over cached rows [latent (rank) | rotated key part (rot_dim)]: a query head is [dim | rot_dim] values, its last rot_dim turned like the key's, score = (q . W_uk c + q_rot . k_rot) * scale.
+ * sink_dev nullable (a plain soft-max); gate_dev (nullable): head h's output times gate[t][h] (gate_act PI_ACT_SIGMOID while the values are still raw) */
+PI_API int pi_op_latent_attention_rot(const float * q_dev, int64_t q_stride, const float * cache_dev, const uint32_t * mask_dev, const pi_weight * w_uk, const pi_weight * w_uv, const float * sink_dev, const float * gate_dev,
+                                      int64_t gate_stride, int gate_act, float scale, int heads, int dim, int rot_dim, int vdim, int rank, const void * rotary_table, const int32_t * pos_dev, int n_tok, int n_kv,
+                                      float * scratch_dev, size_t scratch_floats, float * out_dev, int64_t out_stride, const int32_t * dyn_dev, void * stream);
+PI_API size_t pi_op_latent_attention_rot_scratch_floats(int heads, int rank, int rot_dim, int n_tok, int n_kv);
+
 #ifdef __cplusplus
 }
 #endif

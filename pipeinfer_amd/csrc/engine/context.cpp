@@ -44,6 +44,7 @@ llama_context::~llama_context() {
     pi_free(abort_dev);
     void * bufs[] = { cell_pos, hist, h_out2, h_out3, x_pair, ssd_dt, lat_cache, rec_state, rec_dev, pair_dev, h_in, h_att, h_out, moe_w, moe_up, moe_dn, lat_scratch, rec_scratch, moe_sel, moe_idx, k_cache, v_cache, x, x2, nx, nx2, qkv, att, up, gate, logits_dev, q16, q8a, q8b, q8c, tokens_dev, pos_dev, dyn_dev, mask_dev, topk_ids_dev, topk_vals_dev, topk_sum_dev, topk_scratch_dev };
     for (void * b : bufs) pi_free(b);
+    for (auto & kv : window_masks) pi_free(kv.second);
     if (rope) pi_rope_table_free(rope);
     if (stream) (void) hipStreamDestroy(stream);
 }
@@ -69,6 +70,7 @@ size_t decode_alg_bytes(const llama_context * ctx, int n_tok, int n_kv) {
     }
     size_t b = ctx->alg_w_fixed + ctx->alg_w_per_tok * (size_t) n_tok;
     b += (size_t) n_kv * kv_bytes_per_cell(ctx) + (size_t) n_tok * kv_bytes_per_cell(ctx);
+    for (const auto & l : hp.hybrid) if (l.kv_from >= 0) b += (size_t) n_kv * 4 * hp.hybrid[(size_t) l.kv_from].cell_floats();      // (keys and values read once more, by a layer that has none)
     b += (size_t) 8 * hp.n_embd * n_tok;
     if (ctx->is_last) b += (size_t) 4 * hp.n_vocab * n_tok;
     return b;
@@ -89,6 +91,8 @@ bool context_prepare(llama_context * ctx, std::string & err) {
     if (ctx->seg_layers > 0 && !context_precapture(ctx, std::max(8, ctx->coalesce_max.load()))) { ctx->last_error = "graph capture of the narrow pass widths failed: " + ctx->last_error; err = ctx->last_error; return false; }
     return true;
 }
+// rows that start on 16-byte boundaries when they lie one after the other
+static int row_of_4(int n) { return (n + 3) / 4 * 4; }
 // device state of a hybrid model: latent caches and recurrent states at per-layer offsets, fp32 scratch rows for the widest layer
 static bool context_prepare_hybrid(llama_context * ctx, std::string & err) {
     llama_model * m = ctx->model;
@@ -109,6 +113,26 @@ static bool context_prepare_hybrid(llama_context * ctx, std::string & err) {
     if (hp.n_recurrent() > 0 || hp.pair_buckets > 0) ctx->slots.reset(new state_slots(std::max(1, ctx->n_state_slots)));      // (the previous token of a pair embedding is per-sequence state as well)
     for (size_t i = 0; i < hp.hybrid.size(); i++) {
         const pi_hybrid_layer & H = hp.hybrid[i];
+        if (hp.streams > 0) {                                                  // scratch rows as forward_stream_blocks lays them out
+            if (H.cache_index >= 0) { ctx->lat_off[i] = lat; lat += (size_t) ctx->n_ctx * H.cell_floats(); }
+            if (H.kv_from >= 0) ctx->lat_off[i] = ctx->lat_off[(size_t) H.kv_from];
+            if (H.state_index >= 0) { ctx->rec_off[i] = rec; rec += (size_t) ctx->slots->size() * H.state_floats(); }
+            in_w = std::max(in_w, std::max((size_t) row_of_4(H.in_rows()), (size_t) 3 * H.ff));
+            if (H.mixer == PI_MIXER_MEMORY) {
+                const pi_memory & M = H.memory;
+                att_w = std::max(att_w, (size_t) M.heads * (2 * M.vdim + 1) + (size_t) 3 * M.heads + 4);
+                ctx->rec_scratch_floats = std::max(ctx->rec_scratch_floats, pi_op_linear_attention_scratch_floats(M.heads, M.dim, M.vdim + 1, nb, ctx->slots->size()));
+            } else if (H.mixer == PI_MIXER_WINDOW_ATTENTION) {
+                att_w = std::max(att_w, (size_t) H.left.heads * (H.left.dim + H.left.vdim));
+                ctx->lat_scratch_floats = std::max(ctx->lat_scratch_floats, pi_op_window_attention_scratch_floats(H.left.heads, H.left.vdim, nb));
+            } else {
+                att_w = std::max(att_w, (size_t) row_of_4(H.latent.q_rank) + (size_t) H.heads * (H.dim + H.latent.rot_dim) + (size_t) H.heads * H.vdim + 4);
+                ctx->lat_scratch_floats = std::max(ctx->lat_scratch_floats, pi_op_latent_attention_rot_scratch_floats(H.heads, H.kv_rank, H.latent.rot_dim, nb, ctx->n_ctx));
+                if (H.latent.window > 0) ctx->window_masks[H.latent.window] = nullptr;
+            }
+            positions = true;
+            continue;
+        }
         if (H.mixer == PI_MIXER_CHANNEL_DELTA || H.mixer == PI_MIXER_PARALLEL_SHIFT) {        // scratch rows as forward_post_norm_blocks lays them out
             if (H.mixer == PI_MIXER_CHANNEL_DELTA) {
                 const pi_channel_delta & D = H.delta;
@@ -168,7 +192,7 @@ static bool context_prepare_hybrid(llama_context * ctx, std::string & err) {
         ctx->branch_events.assign(2 * hp.hybrid.size(), nullptr);
         for (hipEvent_t & e : ctx->branch_events) if (hipEventCreateWithFlags(&e, hipEventDisableTiming) != hipSuccess) { err = "hipEventCreate(branch) failed"; return false; }
     }
-    if (!(ctx->x = (float *) dev((size_t) 4 * nb * width)) || !(ctx->nx = (float *) dev((size_t) 4 * nb * width)) || !(ctx->h_out = (float *) dev((size_t) 4 * nb * width)) ||
+    if (!(ctx->x = (float *) dev((size_t) 4 * nb * width * std::max(1, hp.streams))) || !(ctx->nx = (float *) dev((size_t) 4 * nb * width)) || !(ctx->h_out = (float *) dev((size_t) 4 * nb * width)) ||
         !(ctx->h_in = (float *) dev((size_t) 4 * nb * in_w)) || !(ctx->h_att = (float *) dev((size_t) 4 * nb * att_w)) || !(ctx->moe_up = (float *) dev((size_t) 4 * nb * up_w)) ||
         !(ctx->moe_w = (float *) dev((size_t) 4 * nb * sel_w)) || !(ctx->moe_dn = (float *) dev((size_t) 4 * nb * sel_w * width)) || !(ctx->moe_idx = (int32_t *) dev((size_t) 4 * idx_n)) || !(ctx->moe_sel = (int32_t *) dev((size_t) 4 * nb * sel_w)) || (ctx->slots && !(ctx->rec_dev = (int32_t *) dev((size_t) 4 * nb))) || (hp.pair_buckets > 0 && !(ctx->pair_dev = (int32_t *) dev((size_t) 4 * nb))) ||
         !(ctx->tokens_dev = (int32_t *) dev((size_t) 4 * nb)) || !(ctx->pos_dev = (int32_t *) dev((size_t) 4 * nb)) || !(ctx->dyn_dev = (int32_t *) dev((size_t) 4 * (4 + 2 * nb))))
@@ -184,6 +208,7 @@ static bool context_prepare_hybrid(llama_context * ctx, std::string & err) {
     if (pi_op_latent_attention_reserve() != 0 || (hp.n_recurrent() > 0 && (pi_op_linear_attention_reserve() != 0 || pi_op_channel_recurrence_reserve() != 0))) { err = pi_last_error(); return false; }
     ctx->mask_cap_words = (size_t) nb * ((ctx->n_ctx + 31) / 32);
     if (!(ctx->mask_dev = (uint32_t *) dev(ctx->mask_cap_words * 4))) return false;
+    for (auto & kv : ctx->window_masks) if (!(kv.second = (uint32_t *) dev(ctx->mask_cap_words * 4))) return false;
     if (!(ctx->logits_dev = (float *) dev((size_t) 4 * nb * hp.n_vocab)) || !(ctx->topk_ids_dev = (int32_t *) dev((size_t) 4 * nb * 8)) ||
         !(ctx->topk_vals_dev = (float *) dev((size_t) 4 * nb * 8)) || !(ctx->topk_sum_dev = (float *) dev((size_t) 4 * nb)) || !(ctx->topk_scratch_dev = dev(pi_op_topk_scratch_bytes(nb))))
         return false;
@@ -598,12 +623,117 @@ static bool forward_shared_norm_blocks(llama_context * ctx, int n_tok, int n_kv)
     return true;
 }
 
+// Blocks over several residual streams (hp.streams > 0), R(u) = u / sqrt(mean(u^2) + eps):   per sublayer   u = in . X;  y = sublayer(R(u) * w);  X <- mix^T X + out y.
+//   matrix memory      ONE projection [q | k | v | g | i | f] -> the gates' running maximum and factors -> the linear recurrence with the keys' sum as one more value column -> / normaliser, per-head norm,
+//                      * weight * sigmoid(g) -> W_o
+//   attention          ONE projection [q | k | v] (or q alone: another layer's keys and values are read), biases in its epilogue -> q / k divided by their root mean square, query temperature, cache store ->
+//                      soft-max attention -> W_o
+//   latent attention   ONE projection [query latent | key / value latent | rotated key part | gate] -> both latents normed, key part rotated, cache store -> W_uq -> attention over the latents (W_uk folded
+//                      into the query, W_uv applied behind; the window is in the mask rows) * sigmoid(gate) per head -> W_o
+//   feed-forward       [silu(gate) | up] -> product -> down
+// A sublayer ends in ONE row kernel (pi_op_hyper_step): the streams' step, the next sublayer's input and its norm; behind the last one the sum of the streams and the model's norm.
+static bool forward_memory(llama_context * ctx, const pi_hybrid_layer & H, const pi_hybrid_weights & W, size_t il, const float * N, int n_tok) {
+    hipStream_t s = ctx->stream;
+    const pi_memory & M = H.memory;
+    const int width = ctx->model->hparams.n_embd, ex = ctx->exact, nb = ctx->n_batch, n_slots = ctx->slots->size();
+    const int64_t pw = row_of_4(M.in_rows()), hd = (int64_t) M.heads * M.dim, hv = (int64_t) M.heads * M.vdim, hv1 = hv + M.heads;
+    float * P = ctx->h_in, * O = ctx->h_att, * Z = O + (size_t) nb * hv, * forget = Z + (size_t) nb * hv1, * put = forget + (size_t) nb * M.heads, * flo = put + (size_t) nb * M.heads;
+    float * S = ctx->rec_state + ctx->rec_off[il], * m_run = S + (size_t) n_slots * M.matrix_floats();
+    OP_OK(pi_op_dense(W.w_in, N, width, n_tok, P, pw, PI_ACT_NONE, pw, PI_ACT_NONE, ex, s));
+    OP_OK(pi_op_memory_gates(P + 2 * hd + 2 * hv, P + 2 * hd + 2 * hv + M.heads, pw, W.gate_bias, W.gate_bias + M.heads, M.cap, M.heads, m_run, ctx->rec_dev, n_tok, forget, put, flo, s));
+    OP_OK(pi_op_linear_attention_keysum(P, P + hd, P + 2 * hd, pw, M.heads, M.heads, M.dim, M.vdim, 1, nullptr, forget, put, M.heads, nullptr, S, ctx->rec_dev, n_tok, n_slots, ctx->rec_scratch, ctx->rec_scratch_floats, Z, hv1, s));
+    OP_OK(pi_op_memory_norm(Z, hv1, flo, 1.0f / sqrtf((float) M.dim), 1e-6f, M.heads, M.vdim, ctx->model->hparams.f_norm_rms_eps, W.mix_norm, P + 2 * hd + hv, pw, PI_ACT_SIGMOID, n_tok, O, hv, s));
+    trace(ctx, "mem", (int) il, O, hv, n_tok);
+    OP_OK(pi_op_dense(W.w_o, O, hv, n_tok, ctx->h_out, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
+    return true;
+}
+static bool forward_temp_attention(llama_context * ctx, const pi_hybrid_layer & H, const pi_hybrid_weights & W, size_t il, const float * N, int n_tok, int n_kv) {
+    hipStream_t s = ctx->stream;
+    const pi_gate_attention & A = H.left;
+    const int width = ctx->model->hparams.n_embd, ex = ctx->exact, nb = ctx->n_batch;
+    const bool own = H.kv_from < 0;
+    const int64_t pw = row_of_4(H.in_rows()), hd = (int64_t) A.heads * A.dim, hv = (int64_t) A.heads * A.vdim, gd = (int64_t) A.kv_heads * A.dim;
+    float * P = ctx->h_in, * Q = ctx->h_att, * O = Q + (size_t) nb * hd;
+    float * kc = ctx->lat_cache + ctx->lat_off[il], * vc = kc + (size_t) ctx->n_ctx * gd;
+    OP_OK(pi_op_dense_bias(W.w_in, W.in_bias, N, width, n_tok, P, pw, PI_ACT_NONE, pw, PI_ACT_NONE, ex, s));
+    OP_OK(pi_op_qkv_prepare_temp(P, own ? P + hd : nullptr, own ? P + hd + gd : nullptr, pw, nullptr, nullptr, ctx->model->hparams.f_norm_rms_eps, A.heads, A.kv_heads, A.dim, A.vdim, W.rotary, A.qk_norm, A.pairing,
+                                 A.v_norm ? 1 : 0, A.temp_coef, A.temp_every, ctx->pos_dev, n_tok, Q, hd, kc, vc, ctx->cell_pos, ctx->dyn_dev, s));
+    OP_OK(pi_op_window_attention(Q, hd, kc, vc, ctx->cell_pos, ctx->mask_dev, ctx->pos_dev, nullptr, nullptr, nullptr, 0, PI_ACT_NONE, A.scale, 1.0f, A.weights, A.softcap, A.mask_kind, A.chunk, 0, 0, 0, A.heads, A.kv_heads, A.dim,
+                                 A.vdim, n_tok, n_kv, ctx->lat_scratch, ctx->lat_scratch_floats, O, hv, ctx->dyn_dev, s));
+    trace(ctx, "att", (int) il, O, hv, n_tok);
+    OP_OK(pi_op_dense(W.w_o, O, hv, n_tok, ctx->h_out, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
+    return true;
+}
+static bool forward_latent_window(llama_context * ctx, const pi_hybrid_layer & H, const pi_hybrid_weights & W, size_t il, const float * N, int n_tok, int n_kv) {
+    hipStream_t s = ctx->stream;
+    const pi_latent & A = H.latent;
+    const int width = ctx->model->hparams.n_embd, ex = ctx->exact, nb = ctx->n_batch, R = A.rot_dim;
+    const int64_t pw = row_of_4(H.in_rows()), cw = row_of_4(A.q_rank), qw = (int64_t) H.heads * (H.dim + R), hv = (int64_t) H.heads * H.vdim;
+    float * P = ctx->h_in, * C = ctx->h_att, * Q = C + (size_t) nb * cw, * O = Q + (size_t) nb * qw;
+    float * cache = ctx->lat_cache + ctx->lat_off[il];
+    const uint32_t * mask = A.window > 0 ? ctx->window_masks.at(A.window) : ctx->mask_dev;
+    OP_OK(pi_op_dense(W.w_in, N, width, n_tok, P, pw, PI_ACT_NONE, pw, PI_ACT_NONE, ex, s));
+    OP_OK(pi_op_latent_prepare(P, pw, A.q_rank, W.q_norm, H.kv_rank, W.mix_norm, R, W.rotary, ctx->model->hparams.f_norm_rms_eps, ctx->pos_dev, n_tok, C, cw, cache, ctx->dyn_dev, s));
+    OP_OK(pi_op_dense(W.w_uq, C, cw, n_tok, Q, qw, PI_ACT_NONE, qw, PI_ACT_NONE, ex, s));
+    OP_OK(pi_op_latent_attention_rot(Q, qw, cache, mask, W.w_uk, W.w_uv, nullptr, A.gated ? P + A.q_rank + H.kv_rank + R : nullptr, pw, PI_ACT_SIGMOID, H.scale, H.heads, H.dim, R, H.vdim, H.kv_rank, W.rotary, ctx->pos_dev, n_tok,
+                                     n_kv, ctx->lat_scratch, ctx->lat_scratch_floats, O, hv, ctx->dyn_dev, s));
+    trace(ctx, "lat", (int) il, O, hv, n_tok);
+    OP_OK(pi_op_dense(W.w_o, O, hv, n_tok, ctx->h_out, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
+    return true;
+}
+static bool forward_stream_blocks(llama_context * ctx, int n_tok, int n_kv) {
+    llama_model * m = ctx->model;
+    const pi_hparams & hp = m->hparams;
+    hipStream_t s = ctx->stream;
+    const int width = hp.n_embd, ex = ctx->exact, nb = ctx->n_batch, ns = hp.streams;
+    const float eps = hp.f_norm_rms_eps;
+    const size_t n_layer = hp.hybrid.size();
+    float * X = ctx->x, * N = ctx->nx, * Y = ctx->h_out, * P = ctx->h_in;
+    auto owner = [&](size_t il) -> const pi_hybrid_weights & { return m->hweights[(size_t) hp.hybrid[il].weights]; };
+    for (auto & kv : ctx->window_masks) OP_OK(pi_op_window_mask(ctx->mask_dev, ctx->pos_dev, ctx->cell_pos, kv.first, n_tok, n_kv, kv.second, ctx->dyn_dev, s));
+    OP_OK(pi_op_embed(m->tok_embd, ctx->tokens_dev, n_tok, hp.embed_scale, Y, s));
+    OP_OK(pi_op_hyper_step(Y, width, 0, ns, nullptr, 0, nullptr, nullptr, owner(0).hc_in[0], owner(0).norm1, eps, width, n_tok, X, N, width, s));       // every stream starts as the embedding row
+    for (size_t il = 0; il < n_layer; il++) {
+        const pi_hybrid_layer & H = hp.hybrid[il];
+        const pi_hybrid_weights & W = owner(il);
+        const bool last = il + 1 == n_layer;
+        // the streams' step of sublayer q and the input of what comes next (the next layer's mixer; behind the last layer the plain sum of the streams and the model's norm)
+        auto step_out = [&](int q) {
+            const float * in_next = last ? nullptr : owner(il + 1).hc_in[0], * w_next = last ? m->output_norm : owner(il + 1).norm1;
+            return pi_op_hyper_step(X, (int64_t) ns * width, width, ns, Y, width, W.hc_mix[q], W.hc_out[q], in_next, w_next, eps, width, n_tok, last && !trace_enabled() ? nullptr : X, N, width, s);
+        };
+        bool ok = false;
+        switch (H.mixer) {
+            case PI_MIXER_MEMORY:           ok = forward_memory(ctx, H, W, il, N, n_tok); break;
+            case PI_MIXER_WINDOW_ATTENTION: ok = forward_temp_attention(ctx, H, W, il, N, n_tok, n_kv); break;
+            case PI_MIXER_LATENT_ATTENTION: ok = forward_latent_window(ctx, H, W, il, N, n_tok, n_kv); break;
+            default: ctx->last_error = "blocks over residual streams are built for the matrix-memory, attention and latent-attention mixers";
+        }
+        if (!ok) return false;
+        if (!H.has_mlp) OP_OK(step_out(0));
+        else {
+            OP_OK(pi_op_hyper_step(X, (int64_t) ns * width, width, ns, Y, width, W.hc_mix[0], W.hc_out[0], W.hc_in[1], W.norm2, eps, width, n_tok, X, N, width, s));
+            const int ff = H.ff;
+            float * G = P + (size_t) nb * 2 * ff;
+            OP_OK(pi_op_dense(W.ff_up, N, width, n_tok, P, 2 * (int64_t) ff, PI_ACT_SILU, ff, PI_ACT_NONE, ex, s));
+            OP_OK(pi_op_glu_mul(P, 2 * (int64_t) ff, ff, n_tok, G, ff, s));
+            OP_OK(pi_op_dense(W.ff_down, G, ff, n_tok, Y, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
+            OP_OK(step_out(1));
+        }
+        trace(ctx, "lout", (int) il, X, (int64_t) ns * width, n_tok);
+    }
+    OP_OK(pi_op_dense(m->output, N, width, n_tok, ctx->logits_dev, hp.n_vocab, PI_ACT_NONE, hp.n_vocab, PI_ACT_NONE, ex, s));
+    OP_OK(pi_op_topk(ctx->logits_dev, hp.n_vocab, n_tok, 8, ctx->topk_ids_dev, ctx->topk_vals_dev, ctx->topk_sum_dev, ctx->topk_scratch_dev, s));
+    return true;
+}
+
 static bool forward_hybrid(llama_context * ctx, int n_tok, int n_kv) {
     llama_model * m = ctx->model;
     const pi_hparams & hp = m->hparams;
     if (hp.pre_post_norm) return forward_pre_post_blocks(ctx, n_tok, n_kv);
     if (hp.post_norm) return forward_post_norm_blocks(ctx, n_tok, n_kv);
     if (hp.shared_tanh_norm) return forward_shared_norm_blocks(ctx, n_tok, n_kv);
+    if (hp.streams > 0) return forward_stream_blocks(ctx, n_tok, n_kv);
     hipStream_t s = ctx->stream;
     const int width = hp.n_embd, ex = ctx->exact;
     const float eps = hp.f_norm_rms_eps, rm = hp.residual_mult;

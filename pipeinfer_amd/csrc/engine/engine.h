@@ -36,7 +36,9 @@ enum pi_arch { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_BAICHUAN = 2, PI_A
                PI_ARCH_VIKARAX = 10 /* hybrid as well: layer norms before and after every sublayer, a learned average over depth, mixers of two parallel branches */,
                PI_ARCH_RAFUSUN = 11 /* hybrid as well: the norm AFTER the sum (x <- R(alpha x + ls * sublayer(x)) * w), a hashed pair embedding, delta-rule and attention + time-mix mixers */,
                PI_ARCH_RAREVIK = 12 /* hybrid as well: ONE tanh norm per layer that mixer and feed-forward both read (x <- x + mixer(shift(h)) + ff(h)), a run of layers repeated with the same tensors,
-                                       sliding-window attention with pooled far blocks and a learned sink, or with a per-head output gate; clipped gated experts behind a top-logit router */ };
+                                       sliding-window attention with pooled far blocks and a learned sink, or with a per-head output gate; clipped gated experts behind a top-logit router */,
+               PI_ARCH_RERIZEN = 13 /* hybrid as well: the residual is several streams mixed by small learned matrices around every sublayer; mixers: a normalised matrix memory with exponential gates,
+                                       attention with query temperatures (keys and values of its own or another layer's), latent attention behind a query latent with a rotated part and a window */ };
 
 // what the reference's build_* functions differ in (llama.cpp:3985-4104 baichuan, 4229-4327 starcoder, 4540-4630 refact, 4632-4725 bloom, 4727-4825 mpt, 4827-4939 stablelm)
 struct pi_block {
@@ -52,13 +54,16 @@ struct pi_block {
 
 // One layer of a hybrid model.  The mixer is one of the mechanisms below, each with its sizes and constants as the model's description gives them; the feed-forward is a
 // mixture of experts (or absent).  A layer may use another layer's tensors (`weights`) while keeping a cache / state of its own.
-enum pi_mixer_kind { PI_MIXER_LATENT_ATTENTION = 0,   // keys / values are up-projections of one cached low-rank latent, no positions, causal, soft-max with a per-head sink
+enum pi_mixer_kind { PI_MIXER_LATENT_ATTENTION = 0,   // keys / values are up-projections of one cached low-rank latent, causal, soft-max; with a per-head sink, or (pi_latent) queries behind a latent of their own, a rotated part,
+                                                      // a sliding window and a per-head sigmoid gate
                      PI_MIXER_LIGHTNING = 1,          // linear attention with a per-head decay: a [dim][vdim] state per head and sequence
                      PI_MIXER_PARALLEL = 2,           // two branches that read the same input, summed with fixed factors: chunked sigmoid attention (pi_gate_attention) + a selective recurrence (pi_ssd)
                      PI_MIXER_CHANNEL_DELTA = 3,      // gated delta rule with a decay per key channel behind short convolutions (pi_channel_delta)
                      PI_MIXER_PARALLEL_SHIFT = 4,     // two branches, each RMS-normed over the width, averaged: chunked soft-max attention (pi_gate_attention) + time mixing with a token shift (pi_time_mix)
+                     PI_MIXER_MEMORY = 6,             // normalised matrix memory with exponential gates (pi_memory): a [dim][vdim + 1] state and a running maximum per head and sequence
                      PI_MIXER_WINDOW_ATTENTION = 5 }; // soft-max attention over a sliding window of positions (pi_gate_attention with mask_kind = PI_MASK_WINDOW), optionally: a short convolution behind the projections, one pooled
-                                                      // key / value per block of positions that has left the window, a learned sink, a per-head sigmoid gate; reads the layer's token-shifted input
+                                                      // key / value per block of positions that has left the window, a learned sink, a per-head sigmoid gate, a query temperature; reads what the layer's block hands it
+                                                      // (a token-shifted input, a normed mix of streams); may read another layer's keys and values (kv_from)
 // attention with grouped key / value heads, normed and partly rotated q / k, unit-norm values, un-normalised sigmoid weights inside chunks of positions, a per-head output gate
 // (weights / softcap / gated: the soft-max variants — pi_attention_weights — with a tanh cap on the scores and no output gate)
 // (mask_kind: `chunk` is the size of position blocks that do not see each other, or of a window that slides with the token; pool > 0: every block of `pool` positions wholly behind the window is seen
@@ -67,10 +72,19 @@ enum pi_mixer_kind { PI_MIXER_LATENT_ATTENTION = 0,   // keys / values are up-pr
 struct pi_gate_attention { int heads = 0, kv_heads = 0, dim = 0, vdim = 0, rot_dims = 0, chunk = 0; float rot_base = 10000.0f, scale = 1.0f; int weights = PI_WEIGHTS_SIGMOID; float softcap = 0.0f; bool gated = true;
                            int mask_kind = PI_MASK_CHUNK, pool = 0, conv = 0, qk_norm = PI_QK_NORM_FIRST, pairing = PI_PAIR_HALVES; bool v_norm = true;
                            float rot_factor = 1.0f, rot_low = 1.0f, rot_high = 1.0f; int rot_original = 0;
+                           bool bias = false; float temp_coef = 0.0f; int temp_every = 0;                       // biases of q, k, v; query temperature (pi_op_qkv_prepare_temp)
                            int channels() const { return heads * dim + kv_heads * (dim + vdim); }                                  // [q | k | v]
                            int in_rows() const { return channels() + (gated ? heads : 0); }                                       // [q | k | v | gate]
                            int cell_rows() const { return pool > 0 && chunk > 0 && mask_kind == PI_MASK_WINDOW ? 2 : 1; }          // cache rows per cell: the token's own, and the pooled block it completes
                            size_t conv_floats() const { return conv > 1 ? (size_t) (conv - 1) * channels() : 0; } };
+// what a latent attention has besides heads, dim, vdim, kv_rank and scale: a query latent of q_rank values (0: queries straight from the input), rot_dim rotated dimensions per query head and ONE rotated key
+// part of that size per cell, its angle steps stretched along a ramp (rot_original > 0: pi_rotary_table_create_ramp), a window of positions (0: all), a per-head sigmoid gate, a learned sink
+struct pi_latent { int q_rank = 0, rot_dim = 0, window = 0; bool gated = false, sink = true; float rot_base = 10000.0f, rot_factor = 1.0f, rot_fast = 1.0f, rot_slow = 1.0f; int rot_original = 0; };
+// normalised matrix memory: q, k (heads x dim), v and an output gate (heads x vdim), an input and a forget gate per head, both capped; per sequence and head a [dim][vdim] matrix with the decayed sum of the
+// keys as one more column, and the running maximum of the log gates
+struct pi_memory { int heads = 0, dim = 0, vdim = 0; float cap = 1.0f;
+                   int in_rows() const { return 2 * heads * (dim + vdim) + 2 * heads; }                          // [q | k | v | g | i | f]
+                   size_t matrix_floats() const { return (size_t) heads * dim * (vdim + 1); } size_t state_floats() const { return matrix_floats() + (size_t) heads; } };
 // selective state-space recurrence: a [state][vdim] matrix per head and sequence, B / C shared by the heads of a group, a causal convolution of `conv` taps over x, B, C
 struct pi_ssd { int heads = 0, vdim = 0, state = 0, groups = 0, conv = 0, norm_groups = 1;
                 int inner() const { return heads * vdim; } int channels() const { return inner() + 2 * groups * state; } int in_rows() const { return 2 * inner() + 2 * groups * state + heads; }   // [z | x | B | C | dt]
@@ -87,7 +101,8 @@ struct pi_time_mix { int heads = 0, dim = 0, decay_rank = 0, width = 0;
 enum pi_mlp_kind { PI_MLP_NONE = 0, PI_MLP_MOE_RELU_SQR = 1 /* routed by a soft-max with correction, experts relu(up)^2, identity experts */, PI_MLP_DENSE_RELU_SQR = 2,
                    PI_MLP_MOE_GLU = 3 /* routed by sigmoid scores inside the best groups, experts silu(gate) * up, an optional shared expert */, PI_MLP_DENSE_GEGLU = 4 /* down (gelu_tanh(gate) * up) */,
                    PI_MLP_DENSE_GELU = 5 /* down gelu(up), the erf form */, PI_MLP_MOE_CLIPPED = 6 /* the `top` largest router logits (+ bias), soft-max over those; experts down(g sigmoid(1.702 g) (u + 1)) with
-                                                                                                       g = min(gate, limit), u = clip(up, +-limit); an optional shared expert of the same form times a per-token sigmoid gate */ };
+                                                                                                       g = min(gate, limit), u = clip(up, +-limit); an optional shared expert of the same form times a per-token sigmoid gate */,
+                   PI_MLP_DENSE_SWIGLU = 7 /* down (silu(gate) * up) */ };
 struct pi_hybrid_layer {
     pi_mixer_kind mixer = PI_MIXER_LATENT_ATTENTION;
     int weights = 0;                                  // index of the layer that owns the tensors (its own index unless shared)
@@ -96,19 +111,20 @@ struct pi_hybrid_layer {
     std::vector<float> decay;                         // lightning: per head
     pi_gate_attention left; pi_ssd right; float left_scale = 1.0f, right_scale = 1.0f;      // PI_MIXER_PARALLEL
     pi_channel_delta delta; pi_time_mix shift;                                              // PI_MIXER_CHANNEL_DELTA; PI_MIXER_PARALLEL_SHIFT (beside `left`)
+    pi_latent latent; pi_memory memory; int kv_from = -1;                                   // PI_MIXER_LATENT_ATTENTION; PI_MIXER_MEMORY; PI_MIXER_WINDOW_ATTENTION: the layer whose keys and values it reads (-1: its own)
     bool has_mlp = false; int n_expert = 0, n_identity = 0, top = 0, ff = 0;
     pi_mlp_kind mlp = PI_MLP_NONE; int route_groups = 0, route_keep = 0, shared_ff = 0;     // (has_mlp <=> mlp != PI_MLP_NONE)
     float glu_limit = 0.0f, shared_limit = 0.0f;      // clipped experts: the bound on gate (from above) and up (both sides); 0: none
     int name_index = -1;                              // the layer of the description whose names the tensors carry (a repeated run lists a layer several times; -1: the entry's own index)
     bool loop_entry = false;                          // first layer of a repeated run: x <- W_in [x ; embedding row] in front of it
     int cache_index = -1, state_index = -1;           // ordinal among the layers that keep a per-cell cache / a recurrent state
-    int in_rows() const { return mixer == PI_MIXER_CHANNEL_DELTA ? delta.in_rows() : mixer == PI_MIXER_PARALLEL_SHIFT || mixer == PI_MIXER_WINDOW_ATTENTION ? left.in_rows() : mixer == PI_MIXER_PARALLEL ? left.in_rows() + right.in_rows() : mixer == PI_MIXER_LIGHTNING ? 2 * heads * dim + 2 * heads * vdim : heads * dim + kv_rank; }     // rows of the fused input projection
+    int in_rows() const { return mixer == PI_MIXER_MEMORY ? memory.in_rows() : mixer == PI_MIXER_LATENT_ATTENTION && latent.q_rank > 0 ? latent.q_rank + kv_rank + latent.rot_dim + (latent.gated ? heads : 0) : kv_from >= 0 ? left.heads * left.dim : mixer == PI_MIXER_CHANNEL_DELTA ? delta.in_rows() : mixer == PI_MIXER_PARALLEL_SHIFT || mixer == PI_MIXER_WINDOW_ATTENTION ? left.in_rows() : mixer == PI_MIXER_PARALLEL ? left.in_rows() + right.in_rows() : mixer == PI_MIXER_LIGHTNING ? 2 * heads * dim + 2 * heads * vdim : heads * dim + kv_rank; }     // rows of the fused input projection
     int out_cols() const { return mixer == PI_MIXER_CHANNEL_DELTA ? delta.heads * delta.vdim : mixer == PI_MIXER_WINDOW_ATTENTION ? left.heads * left.vdim : mixer == PI_MIXER_PARALLEL_SHIFT ? std::max(left.heads * left.vdim, shift.inner()) : mixer == PI_MIXER_PARALLEL ? std::max(left.heads * left.vdim, right.inner()) : heads * vdim; }                                                   // widest input of an output projection
-    size_t cell_floats() const { return mixer == PI_MIXER_CHANNEL_DELTA ? 0 : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) left.cell_rows() * left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_PARALLEL || mixer == PI_MIXER_PARALLEL_SHIFT ? (size_t) left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_LATENT_ATTENTION ? (size_t) kv_rank : 0; }   // cached per cell
-    size_t state_floats() const { return mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) shift.width + left.conv_floats() : mixer == PI_MIXER_CHANNEL_DELTA ? delta.state_floats() : mixer == PI_MIXER_PARALLEL_SHIFT ? shift.state_floats() : mixer == PI_MIXER_PARALLEL ? right.state_floats() : mixer == PI_MIXER_LIGHTNING ? (size_t) heads * dim * vdim : 0; }                       // kept per sequence
-    // a layer's per-sequence state has up to two parts, each stored [slots][part]: the recurrence's matrices, then the convolution's last inputs / the previous token's input
+    size_t cell_floats() const { return mixer == PI_MIXER_CHANNEL_DELTA || kv_from >= 0 ? 0 : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) left.cell_rows() * left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_PARALLEL || mixer == PI_MIXER_PARALLEL_SHIFT ? (size_t) left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_LATENT_ATTENTION ? (size_t) kv_rank + latent.rot_dim : 0; }   // cached per cell
+    size_t state_floats() const { return mixer == PI_MIXER_MEMORY ? memory.state_floats() : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) shift.width + left.conv_floats() : mixer == PI_MIXER_CHANNEL_DELTA ? delta.state_floats() : mixer == PI_MIXER_PARALLEL_SHIFT ? shift.state_floats() : mixer == PI_MIXER_PARALLEL ? right.state_floats() : mixer == PI_MIXER_LIGHTNING ? (size_t) heads * dim * vdim : 0; }                       // kept per sequence
+    // a layer's per-sequence state has up to two parts, each stored [slots][part]: the recurrence's matrices, then the convolution's last inputs / the previous token's input / the gates' running maximum
     void state_parts(size_t parts[2]) const {
-        parts[0] = mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) shift.width /* the previous token's normed input */ : mixer == PI_MIXER_CHANNEL_DELTA ? delta.matrix_floats() : mixer == PI_MIXER_PARALLEL_SHIFT ? shift.matrix_floats() : mixer == PI_MIXER_PARALLEL ? (size_t) right.heads * right.state * right.vdim : state_floats();
+        parts[0] = mixer == PI_MIXER_MEMORY ? memory.matrix_floats() : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) shift.width /* the previous token's normed input */ : mixer == PI_MIXER_CHANNEL_DELTA ? delta.matrix_floats() : mixer == PI_MIXER_PARALLEL_SHIFT ? shift.matrix_floats() : mixer == PI_MIXER_PARALLEL ? (size_t) right.heads * right.state * right.vdim : state_floats();
         parts[1] = state_floats() - parts[0];
     }
 };
@@ -127,6 +143,9 @@ struct pi_hybrid_weights {                            // the tensors of a layer 
     // tanh norms: the scalar inside the tanh (one float on the device); window attention: the learned sink per head (`sink`), the token-shift factors (`mu`); clipped experts: the router's bias (`correction`),
     // the shared expert [gate | up | its per-token gate row] (ff_up) and down (ff_down); the repeated run's input matrix [width][2 * width] on the entry layer (w_loop)
     float * norm1_alpha = nullptr; pi_weight * w_loop = nullptr;
+    // residual streams: per sublayer the factors of its input [streams], of its result [streams] and the mixing matrix [from][to]; memory: w_in = rows [q | k | v | g | i | f], the gates' biases [i | f]
+    // (gate_bias); attention: the biases of its input rows (in_bias); latent attention: w_in = rows [dq | dkv | g], w_uq, the query latent's norm (q_norm)
+    float * hc_in[2] = { nullptr, nullptr }, * hc_out[2] = { nullptr, nullptr }, * hc_mix[2] = { nullptr, nullptr }, * gate_bias = nullptr, * in_bias = nullptr; pi_weight * w_uq = nullptr;
     pi_weight * w_a2 = nullptr, * w_g2 = nullptr, * w_r = nullptr, * w_k = nullptr, * w_v = nullptr, * w_g = nullptr, * w_w1 = nullptr, * w_w2 = nullptr, * w_o2 = nullptr;
     bool loaded = false;
 };
@@ -147,7 +166,9 @@ struct pi_hparams {
     bool post_norm = false; float post_alpha = 1.0f; int pair_buckets = 0, pair_mul_prev = 0, pair_mul_cur = 0;
     // ... or ONE norm per layer, tanh(alpha x) * w + b, whose output the mixer (token-shifted) and the feed-forward both read: x <- x + mixer(shift(h)) + ff(h)
     bool shared_tanh_norm = false;
-    bool hybrid_arch() const { return arch == PI_ARCH_FASOVIK || arch == PI_ARCH_VIKARAX || arch == PI_ARCH_RAFUSUN || arch == PI_ARCH_RAREVIK; }
+    // ... or `streams` copies of the residual, mixed around every sublayer: u = in . X -> R(u) * w -> sublayer -> X <- mix^T X + out y; the logits times logit_scale
+    int streams = 0; float logit_scale = 1.0f;
+    bool hybrid_arch() const { return arch == PI_ARCH_FASOVIK || arch == PI_ARCH_VIKARAX || arch == PI_ARCH_RAFUSUN || arch == PI_ARCH_RAREVIK || arch == PI_ARCH_RERIZEN; }
     int n_latent() const { int n = 0; for (const auto & l : hybrid) n += l.cache_index >= 0; return n; }
     int n_recurrent() const { int n = 0; for (const auto & l : hybrid) n += l.state_index >= 0; return n; }
     int head_dim() const { return n_embd / n_head; }
@@ -261,6 +282,7 @@ struct llama_context {
     // hybrid models: latent cache [cells][kv_rank] fp32 per latent-attention layer (cells = the kv_cells table above), recurrent states [slots][heads][dim][vdim] fp32 per
     // lightning layer (slots = state_slots), both at per-layer offsets into one allocation each
     float * lat_cache = nullptr, * rec_state = nullptr; std::vector<size_t> lat_off, rec_off;
+    std::map<int, uint32_t *> window_masks;                   // latent attention in windows: the pass's mask rows restricted to a window, per window size
     int32_t * cell_pos = nullptr;                             // position of every cell's token, on the device (mixers that look at positions besides the mask: chunks)
     // a mixer's two branches do not depend on each other between the in- and the out-projection: with PI_BRANCH_STREAMS=1 the second one runs on a stream of its own (forked and joined
     // by events, inside the captured graph as well as in eager launches) so that its small dependent kernels overlap the first one's

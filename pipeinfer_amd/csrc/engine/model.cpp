@@ -41,7 +41,7 @@ llama_model::~llama_model() {
     }
     for (auto & w : hweights) { pi_weight_free(w.w_in); pi_weight_free(w.w_uk); pi_weight_free(w.w_uv); pi_weight_free(w.w_o); pi_weight_free(w.router); pi_weight_free(w.e_up); pi_weight_free(w.e_down);
                                 pi_weight_free(w.ff_up); pi_weight_free(w.ff_down);
-                                for (pi_weight * x : { w.w_a2, w.w_g2, w.w_r, w.w_k, w.w_v, w.w_g, w.w_w1, w.w_w2, w.w_o2 }) pi_weight_free(x);
+                                for (pi_weight * x : { w.w_a2, w.w_g2, w.w_r, w.w_k, w.w_v, w.w_g, w.w_w1, w.w_w2, w.w_o2, w.w_loop, w.w_uq }) pi_weight_free(x);
                                 if (w.rotary) pi_rotary_table_free(w.rotary); }
     for (void * t : retired_tables) pi_rotary_table_free(t);
     pi_weight_free(tok_embd); pi_weight_free(output); pi_weight_free(pos_embd); pi_weight_free(pair_embd);
@@ -196,6 +196,11 @@ size_t llama_model::stage_weight_bytes(int l0, int l1, bool first, bool last, in
                 b += 4 * 4 * w + (H.has_mlp ? 6 * (size_t) H.ff * w : 0);
                 continue;
             }
+            if (hparams.streams > 0) {                                         // the projections and their biases, the up-projections of the latents, the norms' vectors, the dense feed-forward
+                b += 2 * ((size_t) H.in_rows() + H.out_cols()) * w + 4 * (size_t) (H.has_mlp ? 2 : 1) * w + (H.has_mlp ? 6 * (size_t) H.ff * w : 0);
+                if (H.mixer == PI_MIXER_LATENT_ATTENTION) b += 2 * (size_t) H.heads * ((size_t) H.latent.q_rank * (H.dim + H.latent.rot_dim) + (size_t) H.kv_rank * (H.dim + H.vdim));
+                continue;
+            }
             if (H.mixer == PI_MIXER_WINDOW_ATTENTION) {                        // the projections, the norm's and the shift's vectors, the convolution taps, the feed-forward a token uses, a repeated run's input matrix
                 b += 2 * ((size_t) H.in_rows() + (size_t) H.left.heads * H.left.vdim) * w + 4 * 4 * w + 4 * (size_t) H.left.channels() * H.left.conv + (H.loop_entry ? 4 * w * w : 0);
                 if (H.mlp == PI_MLP_DENSE_GELU) b += 4 * (size_t) H.ff * w;
@@ -320,7 +325,7 @@ extern "C" enum llama_vocab_type llama_vocab_type(const struct llama_model * m) 
 extern "C" uint64_t llama_model_size(const struct llama_model * m) { return m->n_bytes; }
 extern "C" uint64_t llama_model_n_params(const struct llama_model * m) { return m->n_elements; }
 extern "C" int llama_model_desc(const struct llama_model * m, char * buf, size_t n) {
-    static const char * names[] = { "llama", "falcon", "baichuan", "starcoder", "refact", "bloom", "mpt", "stablelm", "persimmon", "fasovik", "vikarax", "rafusun", "rarevik" };
+    static const char * names[] = { "llama", "falcon", "baichuan", "starcoder", "refact", "bloom", "mpt", "stablelm", "persimmon", "fasovik", "vikarax", "rafusun", "rarevik", "rerizen" };
     return snprintf(buf, n, "%s %s", names[m->hparams.arch], m->name.c_str());
 }
 

@@ -20,6 +20,11 @@
 // scale, rot.dims / rot.base / rot.scaling.{factor, low, high, original}, mask.size } }, mlp: null | { kind: "dense", ff } | { kind: "moe", expert.ff / expert.limit, router.experts / router.top,
 // shared.ff / shared.limit }.  Tensors: embed, loop.in, final.norm (+ .b, .alpha), l<i>.norm1 (+ .b, .alpha), l<i>.shift, l<i>.mix.{q, k, v, o} with {q.conv, k.conv, v.conv, q.norm, k.norm, sink} or {g},
 // l<i>.mlp.{up, down} or l<i>.mlp.{router, router.b, e<k>.{gate, up, down}, shared.{gate, up, down, sg}}.
+//
+// Rerizen (same files, other keys): vocab, width, streams, norm.eps, logit_scale, layers[]: { type: "mlstm", mixer: { heads, dim, vdim, gate_cap } } or { type: "attention", mixer: { heads, kv_heads, dim, vdim, scale,
+// q_temp.coef / q_temp.every, kv_from (optional: the layer whose keys and values it reads) } } or { type: "latent_attention", mixer: { heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot.dims / rot.base /
+// rot.scaling.{factor, original, fast, slow}, mask.size } }, mlp: null | { kind: "dense", ff }.  Tensors: embed, head, final.norm, l<i>.norm1 / norm2, l<i>.hc1 / hc2.{in, out, mix}, l<i>.mix.{q, k, v, g, o, norm, i, i.b,
+// f, f.b} or l<i>.mix.{q, k, v (+ .b), o} or l<i>.mix.{dq, dq.norm, uq, dkv, dkv.norm, uk, uv, g, o}, l<i>.mlp.{gate, up, down}.
 #include "engine.h"
 #include "json.h"
 
@@ -116,11 +121,11 @@ struct loader {
         if (!t) return nullptr;
         return vector_f32({ bf16_to_f32(((const uint16_t *) t->data)[0]) });
     }
-    float * vector(const std::string & name, int64_t n) {
+    float * vector(const std::string & name, int64_t n, float mult = 1.0f) {
         const pi::st_tensor * t = get(name, { n });
         if (!t) return nullptr;
         std::vector<float> v((size_t) n);
-        for (int64_t i = 0; i < n; i++) v[(size_t) i] = bf16_to_f32(((const uint16_t *) t->data)[i]);
+        for (int64_t i = 0; i < n; i++) v[(size_t) i] = bf16_to_f32(((const uint16_t *) t->data)[i]) * mult;
         return vector_f32(v);
     }
 };
@@ -344,6 +349,96 @@ static bool read_rarevik_config(const pi::json & cfg, pi_hparams & hp, std::stri
     return true;
 }
 
+// Rerizen: several residual streams mixed around every sublayer; normalised matrix memories, attention with a query temperature (keys and values of its own or another layer's), latent attention in windows
+static bool read_rerizen_config(const pi::json & cfg, pi_hparams & hp, std::string & what) {
+    using pi::json;
+    double d;
+    if (!num_at(cfg, "norm.eps", d)) { what = "no 'norm.eps'"; return false; }
+    hp.f_norm_eps = hp.f_norm_rms_eps = (float) d;
+    if (!int_at(cfg, "streams", hp.streams) || hp.streams < 1 || hp.streams > PI_MAX_STREAMS) { what = "'streams' must lie between 1 and " + std::to_string(PI_MAX_STREAMS); return false; }
+    if (hp.n_embd > 16384) { what = "'width' above 16384"; return false; }
+    if (!num_at(cfg, "logit_scale", d)) { what = "no 'logit_scale'"; return false; }
+    hp.logit_scale = (float) d; hp.own_head = true;
+    const json * layers = cfg.find("layers");
+    if (!layers || !layers->is_arr() || layers->arr.empty()) { what = "'layers' must be a non-empty list"; return false; }
+    hp.n_layer = (int) layers->arr.size();
+    hp.n_head = hp.n_head_kv = 1; hp.n_ctx_train = 0;
+    int n_cache = 0, n_state = 0;
+    for (int i = 0; i < hp.n_layer; i++) {
+        const json & jl = layers->arr[(size_t) i];
+        const std::string where = "layers[" + std::to_string(i) + "]: ";
+        auto bad = [&](const std::string & w) { what = where + w; return false; };
+        auto given = [&](const char * path) { const json * v = jl.at(path); return v && !v->is_null(); };
+        pi_hybrid_layer H;
+        H.weights = i;
+        const json * type = jl.find("type");
+        if (!type || !type->is_str()) return bad("no 'type'");
+        if (!int_at(jl, "mixer.heads", H.heads) || !int_at(jl, "mixer.dim", H.dim) || !int_at(jl, "mixer.vdim", H.vdim) || H.heads < 1 || H.dim < 1 || H.vdim < 1) return bad("mixer needs positive 'heads', 'dim', 'vdim'");
+        if (type->str == "mlstm") {
+            H.mixer = PI_MIXER_MEMORY;
+            pi_memory & M = H.memory;
+            M.heads = H.heads; M.dim = H.dim; M.vdim = H.vdim;
+            if (!num_at(jl, "mixer.gate_cap", d) || d <= 0) return bad("mlstm needs a positive 'gate_cap'");
+            M.cap = (float) d;
+            if (M.dim > 1024) return bad("mlstm key width above 1024");
+            H.state_index = n_state++;
+        } else if (type->str == "attention") {
+            H.mixer = PI_MIXER_WINDOW_ATTENTION;
+            pi_gate_attention & A = H.left;
+            A.heads = H.heads; A.dim = H.dim; A.vdim = H.vdim;
+            if (!int_at(jl, "mixer.kv_heads", A.kv_heads) || A.kv_heads < 1 || A.heads % A.kv_heads) return bad("attention needs 'kv_heads', a divisor of heads");
+            if (!num_at(jl, "mixer.scale", d)) return bad("attention needs 'scale'");
+            A.scale = (float) d; A.weights = PI_WEIGHTS_SOFTMAX; A.gated = false; A.v_norm = false; A.bias = true; A.mask_kind = PI_MASK_WINDOW;
+            A.qk_norm = PI_QK_NORM_LAST;                                    // (without a rotation the order says nothing; this one needs no weight)
+            if (given("mixer.mask") && (!int_at(jl, "mixer.mask.size", A.chunk) || A.chunk < 1)) return bad("mixer.mask needs a positive 'size'");
+            if (given("mixer.q_temp")) {
+                if (!num_at(jl, "mixer.q_temp.coef", d) || !int_at(jl, "mixer.q_temp.every", A.temp_every) || A.temp_every < 1) return bad("mixer.q_temp needs 'coef' and a positive 'every'");
+                A.temp_coef = (float) d;
+            }
+            if (given("mixer.kv_from")) {
+                if (!int_at(jl, "mixer.kv_from", H.kv_from) || H.kv_from >= i) return bad("'kv_from' must name an earlier layer");
+                const pi_hybrid_layer & J = hp.hybrid[(size_t) H.kv_from];
+                if (J.mixer != PI_MIXER_WINDOW_ATTENTION || J.kv_from >= 0 || J.left.kv_heads != A.kv_heads || J.left.dim != A.dim || J.left.vdim != A.vdim) return bad("'kv_from' must name an attention layer with keys and values of its own, of this layer's sizes");
+            } else H.cache_index = n_cache++;
+        } else if (type->str == "latent_attention") {
+            H.mixer = PI_MIXER_LATENT_ATTENTION;
+            pi_latent & A = H.latent;
+            A.sink = false; A.gated = true;
+            if (!int_at(jl, "mixer.q_rank", A.q_rank) || !int_at(jl, "mixer.kv_rank", H.kv_rank) || A.q_rank < 1 || H.kv_rank < 1 || H.kv_rank > 1024 || !num_at(jl, "mixer.scale", d)) return bad("latent_attention needs positive 'q_rank', 'kv_rank' (at most 1024) and 'scale'");
+            H.scale = (float) d;
+            if (given("mixer.rot_dim") && !int_at(jl, "mixer.rot_dim", A.rot_dim)) return bad("mixer.rot_dim must be an integer");
+            int dims = 0;
+            if (A.rot_dim > 0) {
+                if ((A.rot_dim & 1) || !int_at(jl, "mixer.rot.dims", dims) || dims != A.rot_dim || !num_at(jl, "mixer.rot.base", d) || d <= 0 || d == 1) return bad("latent_attention rotates its whole 'rot_dim' part: an even 'rot_dim', 'rot.dims' equal to it and a positive 'rot.base' other than 1");
+                A.rot_base = (float) d;
+                if (given("mixer.rot.scaling")) {
+                    double f, fast, slow;
+                    if (!num_at(jl, "mixer.rot.scaling.factor", f) || !int_at(jl, "mixer.rot.scaling.original", A.rot_original) || !num_at(jl, "mixer.rot.scaling.fast", fast) || !num_at(jl, "mixer.rot.scaling.slow", slow) ||
+                        f <= 0 || fast <= 0 || slow <= 0 || A.rot_original < 1) return bad("mixer.rot.scaling needs positive 'factor', 'original', 'fast' and 'slow'");
+                    A.rot_factor = (float) f; A.rot_fast = (float) fast; A.rot_slow = (float) slow;
+                }
+            }
+            if (given("mixer.mask") && (!int_at(jl, "mixer.mask.size", A.window) || A.window < 1)) return bad("mixer.mask needs a positive 'size'");
+            H.cache_index = n_cache++;
+        } else return bad("mixer type '" + type->str + "' is unknown (mlstm, attention, latent_attention)");
+        if (jl.has("mlp")) {
+            const json * kind = jl.at("mlp.kind");
+            if (!kind || !kind->is_str() || kind->str != "dense") return bad("feed-forward kind must be 'dense'");
+            if (!int_at(jl, "mlp.ff", H.ff) || H.ff < 1) return bad("a dense mlp needs 'ff'");
+            H.mlp = PI_MLP_DENSE_SWIGLU; H.has_mlp = true;
+        }
+        hp.hybrid.push_back(std::move(H));
+    }
+    return true;
+}
+
+// the rotation table of a layer, over n_pos positions
+static void * rotary_of(const pi_hybrid_layer & H, int n_pos) {
+    if (H.mixer != PI_MIXER_LATENT_ATTENTION) return pi_rotary_table_create_scaled(n_pos, H.left.rot_dims, H.left.rot_base, H.left.rot_factor, H.left.rot_low, H.left.rot_high, H.left.rot_original);
+    const pi_latent & A = H.latent;
+    return A.rot_original > 0 ? pi_rotary_table_create_ramp(n_pos, A.rot_dim, A.rot_base, A.rot_factor, A.rot_original, A.rot_fast, A.rot_slow) : pi_rotary_table_create(n_pos, A.rot_dim, A.rot_base);
+}
+
 }  // namespace
 
 bool llama_model::ensure_loaded_hybrid(int n_positions, std::string & err) {
@@ -354,11 +449,11 @@ bool llama_model::ensure_loaded_hybrid(int n_positions, std::string & err) {
     const int64_t width = hp.n_embd;
     if (!tok_embd) {
         if (!(tok_embd = L.matrix({ { "embed", hp.n_vocab } }, width))) return false;
-        if (!(output_norm = L.vector("final.norm", width))) return false;
+        if (!(output_norm = L.vector("final.norm", width, hp.logit_scale))) return false;                  // (a factor on the logits is a factor on the rows that enter the output matrix)
     }
     if (hp.own_head && !output) {
         if (!(output = L.matrix({ { "head", hp.n_vocab } }, width))) return false;
-        if (!hp.post_norm && !(output_norm_b = L.vector("final.norm.b", width))) return false;
+        if (!hp.post_norm && hp.streams == 0 && !(output_norm_b = L.vector("final.norm.b", width))) return false;
     }
     if (hp.shared_tanh_norm && !output_norm_alpha && (!(output_norm_b = L.vector("final.norm.b", width)) || !(output_norm_alpha = L.scalar("final.norm.alpha")))) return false;
     if (hp.pair_buckets > 0 && !pair_embd && !(pair_embd = L.matrix({ { "bigram", (int64_t) hp.pair_buckets + 1 } }, width))) return false;
@@ -366,12 +461,45 @@ bool llama_model::ensure_loaded_hybrid(int n_positions, std::string & err) {
         const pi_hybrid_layer & H = hp.hybrid[i];
         pi_hybrid_weights & W = hweights[i];
         if (H.weights == (int) i && W.loaded && W.rotary && pi_rotary_table_positions(W.rotary) < n_positions) {        // a later context is longer than the table
-            void * t = pi_rotary_table_create_scaled(n_positions, H.left.rot_dims, H.left.rot_base, H.left.rot_factor, H.left.rot_low, H.left.rot_high, H.left.rot_original);
+            void * t = rotary_of(H, n_positions);
             if (!t) { err = std::string("rotation table: ") + pi_last_error(); return false; }
             retired_tables.push_back(W.rotary); W.rotary = t;
         }
         if (H.weights != (int) i || W.loaded) continue;
         const std::string p = "l" + std::to_string(H.name_index >= 0 ? H.name_index : (int) i) + ".";
+        if (hp.streams > 0) {                                              // per sublayer a norm and the streams' factors
+            const std::string m = p + "mix.";
+            const int n_sub = H.has_mlp ? 2 : 1;
+            for (int q = 0; q < n_sub; q++) {
+                const std::string c = p + (q ? "hc2." : "hc1.");
+                if (!((q ? W.norm2 : W.norm1) = L.vector(p + (q ? "norm2" : "norm1"), width)) || !(W.hc_in[q] = L.vector(c + "in", hp.streams)) || !(W.hc_out[q] = L.vector(c + "out", hp.streams)) ||
+                    !(W.hc_mix[q] = L.vector2(c + "mix", hp.streams, hp.streams))) return false;
+            }
+            const int64_t hd = (int64_t) H.heads * H.dim, hv = (int64_t) H.heads * H.vdim;
+            if (H.mixer == PI_MIXER_MEMORY) {
+                if (!(W.w_in = L.matrix({ { m + "q", hd }, { m + "k", hd }, { m + "v", hv }, { m + "g", hv }, { m + "i", H.heads }, { m + "f", H.heads } }, width))) return false;
+                if (!(W.gate_bias = L.vectors({ { m + "i.b", H.heads }, { m + "f.b", H.heads } }, 0)) || !(W.mix_norm = L.vector(m + "norm", hv))) return false;
+            } else if (H.mixer == PI_MIXER_WINDOW_ATTENTION) {
+                const pi_gate_attention & A = H.left;
+                std::vector<std::pair<std::string, int64_t>> rows = { { m + "q", hd } }, biases = { { m + "q.b", hd } };
+                if (H.kv_from < 0) {
+                    const int64_t gd = (int64_t) A.kv_heads * A.dim, gv = (int64_t) A.kv_heads * A.vdim;
+                    rows.push_back({ m + "k", gd }); rows.push_back({ m + "v", gv }); biases.push_back({ m + "k.b", gd }); biases.push_back({ m + "v.b", gv });
+                }
+                if (!(W.w_in = L.matrix(rows, width)) || (A.bias && !(W.in_bias = L.vectors(biases, 0)))) return false;
+            } else if (H.mixer == PI_MIXER_LATENT_ATTENTION) {
+                const pi_latent & A = H.latent;
+                std::vector<std::pair<std::string, int64_t>> rows = { { m + "dq", A.q_rank }, { m + "dkv", (int64_t) H.kv_rank + A.rot_dim } };
+                if (A.gated) rows.push_back({ m + "g", H.heads });
+                if (!(W.w_in = L.matrix(rows, width)) || !(W.q_norm = L.vector(m + "dq.norm", A.q_rank)) || !(W.mix_norm = L.vector(m + "dkv.norm", H.kv_rank))) return false;
+                if (!(W.w_uq = L.matrix({ { m + "uq", (int64_t) H.heads * (H.dim + A.rot_dim) } }, A.q_rank)) || !(W.w_uk = L.matrix({ { m + "uk", hd } }, H.kv_rank)) || !(W.w_uv = L.matrix({ { m + "uv", hv } }, H.kv_rank))) return false;
+            } else { err = "a block over residual streams has no mixer of kind " + std::to_string((int) H.mixer); return false; }
+            if (H.mixer != PI_MIXER_MEMORY && !(W.rotary = rotary_of(H, std::max(n_positions, 32)))) { err = std::string("rotation table: ") + pi_last_error(); return false; }
+            if (!(W.w_o = L.matrix({ { m + "o", width } }, hv))) return false;
+            if (H.mlp == PI_MLP_DENSE_SWIGLU && (!(W.ff_up = L.matrix({ { p + "mlp.gate", H.ff }, { p + "mlp.up", H.ff } }, width)) || !(W.ff_down = L.matrix({ { p + "mlp.down", width } }, H.ff)))) return false;
+            W.loaded = true;
+            continue;
+        }
         if (hp.shared_tanh_norm) {                                         // one tanh norm per layer; window attention; dense or routed clipped feed-forward
             if (H.mixer != PI_MIXER_WINDOW_ATTENTION) { err = "a block with one shared tanh norm has no mixer of kind " + std::to_string((int) H.mixer); return false; }
             const pi_gate_attention & A = H.left;
@@ -520,14 +648,15 @@ llama_model * load_hybrid_model(const std::string & folder, const llama_model_pa
     else if (arch->str == "Vikarax") hp.arch = PI_ARCH_VIKARAX;
     else if (arch->str == "Rafusun") hp.arch = PI_ARCH_RAFUSUN;
     else if (arch->str == "Rarevik") hp.arch = PI_ARCH_RAREVIK;
-    else return fail("architecture '" + arch->str + "' is not one this engine builds (Fasovik, Vikarax, Rafusun, Rarevik)");
+    else if (arch->str == "Rerizen") hp.arch = PI_ARCH_RERIZEN;
+    else return fail("architecture '" + arch->str + "' is not one this engine builds (Fasovik, Vikarax, Rafusun, Rarevik, Rerizen)");
     m->name = arch->str;
     double d;
     if (!int_at(cfg, "vocab", hp.n_vocab) || !int_at(cfg, "width", hp.n_embd) || hp.n_vocab < 1 || hp.n_embd < 1) return fail("'vocab' and 'width' must be positive integers");
-    if (hp.arch == PI_ARCH_VIKARAX || hp.arch == PI_ARCH_RAFUSUN || hp.arch == PI_ARCH_RAREVIK) {
+    if (hp.arch == PI_ARCH_VIKARAX || hp.arch == PI_ARCH_RAFUSUN || hp.arch == PI_ARCH_RAREVIK || hp.arch == PI_ARCH_RERIZEN) {
         std::string what;
         if (!params.vocab_only && !m->st_file.open(folder + "/model.safetensors", err)) { fprintf(stderr, "llama_load_model_from_file: %s\n", err.c_str()); return nullptr; }
-        if (hp.arch == PI_ARCH_VIKARAX ? !read_vikarax_config(cfg, hp, what) : hp.arch == PI_ARCH_RAREVIK ? !read_rarevik_config(cfg, hp, what) : !read_rafusun_config(cfg, params.vocab_only ? nullptr : &m->st_file, hp, what)) return fail(what);
+        if (hp.arch == PI_ARCH_RERIZEN ? !read_rerizen_config(cfg, hp, what) : hp.arch == PI_ARCH_VIKARAX ? !read_vikarax_config(cfg, hp, what) : hp.arch == PI_ARCH_RAREVIK ? !read_rarevik_config(cfg, hp, what) : !read_rafusun_config(cfg, params.vocab_only ? nullptr : &m->st_file, hp, what)) return fail(what);
         m->hweights.resize((size_t) hp.n_layer);
         if (!params.vocab_only) {
             for (const auto & kv : m->st_file.tensors) { m->n_elements += (uint64_t) kv.second.elements(); m->n_bytes += kv.second.nbytes; }

@@ -1,6 +1,6 @@
 // Dense operators over bfloat16 weight matrices stored [rows][K] as the checkpoint has them (no re-ordering: a row is one contiguous run of K values).
 //
-//   out[t][r] = act(sum_k W[r][k] * in(x[t][k]))          fp32 accumulation, fp32 in and out
+//   out[t][r] = act(sum_k W[r][k] * in(x[t][k]) [+ bias[r]])          fp32 accumulation, fp32 in and out
 //
 // `exact` selects what enters the product: 0 (serving precision) rounds the activations to bfloat16 (nearest even), so a product of two bfloat16 values is exact in fp32 and only the
 // order of the fp32 sum differs between the kernels below; 1 keeps the activations in fp32 (weights widen exactly), every multiply-add a true fp32 fma.
@@ -48,7 +48,7 @@ __global__ void k_embed(const uint16_t * __restrict__ table, int64_t width, int6
 // VW weights per lane and step (8: one 16-byte load, 4: 8 bytes, 1: any K and alignment)
 template <int TT, int VW, bool EXACT>
 __global__ void __launch_bounds__(256) k_dense_rows(const uint16_t * __restrict__ W, int64_t K, int64_t N, const float * __restrict__ X, int64_t xs, int T, float * __restrict__ Y, int64_t ys,
-                                                    int act_a, int64_t rows_a, int act_b, int64_t seg_rows, int64_t seg_off, int seg_last, const int32_t * __restrict__ abort_w) {
+                                                    int act_a, int64_t rows_a, int act_b, const float * __restrict__ bias, int64_t seg_rows, int64_t seg_off, int seg_last, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 0)) return;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int64_t row = (int64_t) blockIdx.x * 4 + wave;
@@ -82,13 +82,13 @@ __global__ void __launch_bounds__(256) k_dense_rows(const uint16_t * __restrict_
     for (int tt = 0; tt < TT; tt++) {
         if (t0 + tt >= T) break;
         const float s = pi_lanes_sum<64>(acc[tt]);
-        if (lane == 0) Y[(int64_t) (t0 + tt) * ys + row] = dn_act(s, act);
+        if (lane == 0) Y[(int64_t) (t0 + tt) * ys + row] = dn_act(bias ? s + bias[row] : s, act);
     }
 }
 
 // 64 tokens x 64 rows per workgroup; K % 8 == 0, 16-byte aligned rows of W and X
 __global__ void __launch_bounds__(256) k_dense_mfma(const uint16_t * __restrict__ W, int64_t K, int64_t N, const float * __restrict__ X, int64_t xs, int T, float * __restrict__ Y, int64_t ys,
-                                                    int act_a, int64_t rows_a, int act_b, const int32_t * __restrict__ abort_w) {
+                                                    int act_a, int64_t rows_a, int act_b, const float * __restrict__ bias, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 1)) return;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int li = lane & 15, kb = lane >> 4;
@@ -125,7 +125,7 @@ __global__ void __launch_bounds__(256) k_dense_mfma(const uint16_t * __restrict_
 #pragma unroll
         for (int r = 0; r < 4; r++) {
             const int64_t row = n0 + j * 16 + kb * 4 + r;
-            if (row < N) Y[(int64_t) tok * ys + row] = dn_act(acc[j][r], row < rows_a ? act_a : act_b);
+            if (row < N) Y[(int64_t) tok * ys + row] = dn_act(bias ? acc[j][r] + bias[row] : acc[j][r], row < rows_a ? act_a : act_b);
         }
 }
 
@@ -133,7 +133,7 @@ __global__ void __launch_bounds__(256) k_dense_mfma(const uint16_t * __restrict_
 // tiles, so one K step of 32 costs it eight 16-byte LDS reads for sixteen MFMAs; the next K step's global loads are in flight while the current one is multiplied.
 // K % 8 == 0, 16-byte aligned rows of W and X.
 __global__ void __launch_bounds__(256) k_dense_mfma_lds(const uint16_t * __restrict__ W, int64_t K, int64_t N, const float * __restrict__ X, int64_t xs, int T, float * __restrict__ Y, int64_t ys,
-                                                        int act_a, int64_t rows_a, int act_b, const int32_t * __restrict__ abort_w) {
+                                                        int act_a, int64_t rows_a, int act_b, const float * __restrict__ bias, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 1)) return;
     __shared__ __attribute__((aligned(16))) uint16_t sw[2][128 * 32], sx[2][128 * 32];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, kb = lane >> 4;
@@ -197,7 +197,7 @@ __global__ void __launch_bounds__(256) k_dense_mfma_lds(const uint16_t * __restr
             const int64_t row = n0 + wr * 64 + a * 16 + kb * 4;
             float v[4];
 #pragma unroll
-            for (int r = 0; r < 4; r++) v[r] = dn_act(acc[a][b][r], row + r < rows_a ? act_a : act_b);
+            for (int r = 0; r < 4; r++) v[r] = dn_act(bias ? acc[a][b][r] + bias[min(row + r, N - 1)] : acc[a][b][r], row + r < rows_a ? act_a : act_b);
             float * dst = Y + (int64_t) tok * ys + row;
             if (row + 3 < N && (ys & 3) == 0 && (((uintptr_t) Y) & 15) == 0) *(float4 *) dst = make_float4(v[0], v[1], v[2], v[3]);
             else for (int r = 0; r < 4; r++) if (row + r < N) dst[r] = v[r];
@@ -215,16 +215,19 @@ extern "C" int pi_op_embed(const pi_weight * w, const int32_t * tokens, int n_to
 static int dense_mfma_min_tokens() { static const int v = getenv("PI_DENSE_MFMA_MIN") ? atoi(getenv("PI_DENSE_MFMA_MIN")) : 16; return v; }
 
 template <int VW, bool EXACT>
-static void launch_rows(const pi_weight * w, const float * x, int64_t xs, int n_tok, float * out, int64_t os, int act_a, int64_t rows_a, int act_b, hipStream_t s, double bytes, int64_t seg_rows = 0, int64_t seg_off = 0, int seg_last = 0) {
+static void launch_rows(const pi_weight * w, const float * x, int64_t xs, int n_tok, float * out, int64_t os, int act_a, int64_t rows_a, int act_b, hipStream_t s, double bytes, const float * bias = nullptr, int64_t seg_rows = 0, int64_t seg_off = 0, int seg_last = 0) {
     const uint16_t * W = (const uint16_t *) w->p0;
     const unsigned gx = (unsigned) ((w->ne1 + 3) / 4);
     const int nt_acct = std::min(n_tok, PI_KT_MAXNT - 1);
-    if (n_tok == 1)      PI_KT_LAUNCH(PI_KT_MATVEC, PI_BF16, nt_acct, bytes, (k_dense_rows<1, VW, EXACT>), dim3(gx, 1), dim3(256), 0, s, W, w->ne0, w->ne1, x, xs, n_tok, out, os, act_a, rows_a, act_b, seg_rows, seg_off, seg_last, pi_abort_word());
-    else if (n_tok <= 4) PI_KT_LAUNCH(PI_KT_MATVEC, PI_BF16, nt_acct, bytes, (k_dense_rows<4, VW, EXACT>), dim3(gx, 1), dim3(256), 0, s, W, w->ne0, w->ne1, x, xs, n_tok, out, os, act_a, rows_a, act_b, seg_rows, seg_off, seg_last, pi_abort_word());
-    else PI_KT_LAUNCH(PI_KT_MATVEC, PI_BF16, nt_acct, bytes, (k_dense_rows<8, VW, EXACT>), dim3(gx, (unsigned) ((n_tok + 7) / 8)), dim3(256), 0, s, W, w->ne0, w->ne1, x, xs, n_tok, out, os, act_a, rows_a, act_b, seg_rows, seg_off, seg_last, pi_abort_word());
+    if (n_tok == 1)      PI_KT_LAUNCH(PI_KT_MATVEC, PI_BF16, nt_acct, bytes, (k_dense_rows<1, VW, EXACT>), dim3(gx, 1), dim3(256), 0, s, W, w->ne0, w->ne1, x, xs, n_tok, out, os, act_a, rows_a, act_b, bias, seg_rows, seg_off, seg_last, pi_abort_word());
+    else if (n_tok <= 4) PI_KT_LAUNCH(PI_KT_MATVEC, PI_BF16, nt_acct, bytes, (k_dense_rows<4, VW, EXACT>), dim3(gx, 1), dim3(256), 0, s, W, w->ne0, w->ne1, x, xs, n_tok, out, os, act_a, rows_a, act_b, bias, seg_rows, seg_off, seg_last, pi_abort_word());
+    else PI_KT_LAUNCH(PI_KT_MATVEC, PI_BF16, nt_acct, bytes, (k_dense_rows<8, VW, EXACT>), dim3(gx, (unsigned) ((n_tok + 7) / 8)), dim3(256), 0, s, W, w->ne0, w->ne1, x, xs, n_tok, out, os, act_a, rows_a, act_b, bias, seg_rows, seg_off, seg_last, pi_abort_word());
 }
 
 extern "C" int pi_op_dense(const pi_weight * w, const float * x, int64_t x_stride, int n_tok, float * out, int64_t out_stride, int act_a, int64_t rows_a, int act_b, int exact, void * stream) {
+    return pi_op_dense_bias(w, nullptr, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, exact, stream);
+}
+extern "C" int pi_op_dense_bias(const pi_weight * w, const float * bias, const float * x, int64_t x_stride, int n_tok, float * out, int64_t out_stride, int act_a, int64_t rows_a, int act_b, int exact, void * stream) {
     if (!w || w->type != PI_BF16) { pi_set_error("pi_op_dense: the weight must be bfloat16"); return -1; }
     if (n_tok <= 0 || w->ne1 <= 0) return 0;
     if (x_stride < w->ne0 || out_stride < w->ne1) { pi_set_error("pi_op_dense: row strides (%lld, %lld) below the matrix's sizes (%lld, %lld)", (long long) x_stride, (long long) out_stride, (long long) w->ne0, (long long) w->ne1); return -1; }
@@ -236,17 +239,17 @@ extern "C" int pi_op_dense(const pi_weight * w, const float * x, int64_t x_strid
     static const int lds_min = getenv("PI_DENSE_LDS_MIN") ? atoi(getenv("PI_DENSE_LDS_MIN")) : 96;
     if (!exact && al16 && n_tok >= lds_min) {
         PI_KT_LAUNCH(PI_KT_MMQ, PI_BF16, std::min(n_tok, PI_KT_MAXNT - 1), bytes, k_dense_mfma_lds, dim3((unsigned) ((w->ne1 + 127) / 128), (unsigned) ((n_tok + 127) / 128)), dim3(256), 0, s,
-                     (const uint16_t *) w->p0, K, w->ne1, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, pi_abort_word());
+                     (const uint16_t *) w->p0, K, w->ne1, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, bias, pi_abort_word());
         PI_CHECK_LAUNCH(); return 0;
     }
     if (!exact && al16 && n_tok >= dense_mfma_min_tokens()) {
         PI_KT_LAUNCH(PI_KT_MMQ, PI_BF16, std::min(n_tok, PI_KT_MAXNT - 1), bytes, k_dense_mfma, dim3((unsigned) ((w->ne1 + 63) / 64), (unsigned) ((n_tok + 63) / 64)), dim3(256), 0, s,
-                     (const uint16_t *) w->p0, K, w->ne1, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, pi_abort_word());
+                     (const uint16_t *) w->p0, K, w->ne1, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, bias, pi_abort_word());
         PI_CHECK_LAUNCH(); return 0;
     }
-    if (al16 && K >= 512) { if (exact) launch_rows<8, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes); else launch_rows<8, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes); }
-    else if (al8)         { if (exact) launch_rows<4, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes); else launch_rows<4, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes); }
-    else                  { if (exact) launch_rows<1, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes); else launch_rows<1, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes); }
+    if (al16 && K >= 512) { if (exact) launch_rows<8, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, bias); else launch_rows<8, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, bias); }
+    else if (al8)         { if (exact) launch_rows<4, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, bias); else launch_rows<4, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, bias); }
+    else                  { if (exact) launch_rows<1, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, bias); else launch_rows<1, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, bias); }
     PI_CHECK_LAUNCH(); return 0;
 }
 
@@ -264,9 +267,9 @@ extern "C" int pi_op_dense_segments(const pi_weight * w, const float * x, int64_
         const bool al8 = K % 4 == 0 && ((uintptr_t) w->p0 % 8) == 0 && ((uintptr_t) x % 16) == 0 && x_stride % 4 == 0 && seg_off % 4 == 0;
         const double bytes = 2.0 * K * w->ne1 + 4.0 * n_tok * (n_seg * K + w->ne1);
         hipStream_t s = (hipStream_t) stream;
-        if (al16 && K >= 512) { if (exact) launch_rows<8, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, seg_rows, seg_off, n_seg - 1); else launch_rows<8, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, seg_rows, seg_off, n_seg - 1); }
-        else if (al8)         { if (exact) launch_rows<4, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, seg_rows, seg_off, n_seg - 1); else launch_rows<4, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, seg_rows, seg_off, n_seg - 1); }
-        else                  { if (exact) launch_rows<1, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, seg_rows, seg_off, n_seg - 1); else launch_rows<1, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, seg_rows, seg_off, n_seg - 1); }
+        if (al16 && K >= 512) { if (exact) launch_rows<8, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, nullptr, seg_rows, seg_off, n_seg - 1); else launch_rows<8, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, nullptr, seg_rows, seg_off, n_seg - 1); }
+        else if (al8)         { if (exact) launch_rows<4, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, nullptr, seg_rows, seg_off, n_seg - 1); else launch_rows<4, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, nullptr, seg_rows, seg_off, n_seg - 1); }
+        else                  { if (exact) launch_rows<1, true>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, nullptr, seg_rows, seg_off, n_seg - 1); else launch_rows<1, false>(w, x, x_stride, n_tok, out, out_stride, act_a, rows_a, act_b, s, bytes, nullptr, seg_rows, seg_off, n_seg - 1); }
         PI_CHECK_LAUNCH(); return 0;
     }
     for (int g = 0; g < n_seg; g++) {                                  // a view of the segment's rows

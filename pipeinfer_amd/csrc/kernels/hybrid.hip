@@ -2,7 +2,8 @@
 // state, router.  Matrices are bfloat16 pi_weights (widened exactly); `exact` = 0 rounds the activations that enter an expert's matrices to bfloat16 as pi_op_dense does.
 //
 //   k_rms_scale          y = x / sqrt(mean(x^2) + eps) * (w + w_offset) [* gate];  out = [residual +] mult * y;  rows may be written into the cache cells of the pass
-//   k_linear_attention   per head S <- lambda * S + k v^T, o = S^T q over a run of tokens of one sequence; S lives in HBM per (slot, head) between calls
+//   k_linear_attention   per head S <- lambda * S + k v^T, o = S^T q over a run of tokens of one sequence; S lives in HBM per (slot, head) between calls; optionally with a value column of
+//                        ones behind the others (the running sum of keys a normalised memory divides by)
 //   k_latent_attention   attention over a shared low-rank latent c: the key up-projection is folded into the query (q~ = W_uk^T q), the value up-projection applied to the
 //                        probability-weighted sum of latents — the cache is read once for all heads of a tile and K / V are never materialised; soft-max with a sink term
 //   k_norm_chain(_reg)   y = ((ca * a + cb * b) - mean) / sqrt(variance + eps) * w + bias;  out = [residual +] y   (layer norm of one input or of the weighted sum of two), and
@@ -484,7 +485,7 @@ static __device__ __forceinline__ bool la_find_piece(const int * recs, int n_tok
     return false;
 }
 template <int DPT>
-__global__ void __launch_bounds__(256) k_linear_attention(const float * __restrict__ q, const float * __restrict__ k, const float * __restrict__ v, int64_t stride, int heads, int hpg, int dim, int vdim, int R,
+__global__ void __launch_bounds__(256) k_linear_attention(const float * __restrict__ q, const float * __restrict__ k, const float * __restrict__ v, int64_t stride, int heads, int hpg, int dim, int vdim, int vstored, int R,
                                                           const float * __restrict__ decay, const float * __restrict__ tdecay, const float * __restrict__ tscale, int64_t tds, const float * __restrict__ skip,
                                                           float * __restrict__ state, const int32_t * __restrict__ rec, int n_tok, int mode, float * __restrict__ scratch,
                                                           float * __restrict__ out, int64_t os, const int32_t * __restrict__ abort_w) {
@@ -537,7 +538,7 @@ __global__ void __launch_bounds__(256) k_linear_attention(const float * __restri
         }
         for (int idx = tid; idx < nt * cols; idx += blockDim.x) {
             const int tt = idx / cols, jj = blockIdx.y * cols + idx % cols;
-            vt[idx] = jj < vdim ? v[(int64_t) (first + t0 + tt) * stride + (int64_t) h * vdim + jj] : 0.0f;
+            vt[idx] = jj < vstored ? v[(int64_t) (first + t0 + tt) * stride + (int64_t) h * vstored + jj] : jj < vdim ? 1.0f : 0.0f;      // (a column the values do not have: ones)
         }
         __syncthreads();
         if (mode == 1) {                                              // the state only
@@ -649,15 +650,29 @@ extern "C" int pi_op_linear_attention(const float * q, const float * k, const fl
 extern "C" int pi_op_linear_attention_ex(const float * q, const float * k, const float * v, int64_t stride, int heads, int qk_heads, int dim, int vdim, const float * decay_dev, const float * tdecay_dev,
                                          const float * tscale_dev, int64_t t_stride, const float * skip_dev, float * state_dev, const int32_t * rec_dev, int n_tok, int max_segments, float * scratch_dev,
                                          size_t scratch_floats, float * out, int64_t out_stride, void * stream) {
+    return pi_op_linear_attention_keysum(q, k, v, stride, heads, qk_heads, dim, vdim, 0, decay_dev, tdecay_dev, tscale_dev, t_stride, skip_dev, state_dev, rec_dev, n_tok, max_segments, scratch_dev, scratch_floats, out, out_stride, stream);
+}
+extern "C" int pi_op_linear_attention_keysum(const float * q, const float * k, const float * v, int64_t stride, int heads, int qk_heads, int dim, int value_cols, int key_sum, const float * decay_dev, const float * tdecay_dev,
+                                             const float * tscale_dev, int64_t t_stride, const float * skip_dev, float * state_dev, const int32_t * rec_dev, int n_tok, int max_segments, float * scratch_dev,
+                                             size_t scratch_floats, float * out, int64_t out_stride, void * stream) {
     if (n_tok <= 0) return 0;
+    const int vdim = value_cols + (key_sum ? 1 : 0);                   // columns of the state and of an output row per head
     if (qk_heads < 1 || heads % qk_heads) { pi_set_error("pi_op_linear_attention: %d heads do not divide over %d query / key heads", heads, qk_heads); return -1; }
     if (!decay_dev && !tdecay_dev) { pi_set_error("pi_op_linear_attention: neither per-head nor per-token decays were given"); return -1; }
     const int hpg = heads / qk_heads;
-    if (dim <= 0 || vdim <= 0 || heads <= 0 || dim > 1024) { pi_set_error("pi_op_linear_attention: head sizes %d x %d outside the kernel's range (key width <= 1024)", dim, vdim); return -1; }
+    if (dim <= 0 || value_cols <= 0 || heads <= 0 || dim > 1024) { pi_set_error("pi_op_linear_attention: head sizes %d x %d outside the kernel's range (key width <= 1024)", dim, vdim); return -1; }
     if (max_segments > LA_MAXRUNS) { pi_set_error("pi_op_linear_attention: at most %d sequences in a pass", LA_MAXRUNS); return -1; }
     const int dpt = dim <= 8 ? 8 : dim <= 16 ? 16 : 32;                // state values a thread keeps in registers (more would spill in the token loop)
     int R = 1; while (R * dpt < dim) R *= 2;
     int threads = std::min(256, (vdim * R + 63) / 64 * 64);
+    if (key_sum && R <= 64) {                                          // one column more than a round number: blocks of the size that leaves the fewest lanes without a column
+        int best = 1 << 30;
+        const int b0 = (vdim * R + 255) / 256;
+        for (int b = b0; b < b0 + 8; b++) {
+            const int waves = ((vdim + b - 1) / b * R + 63) / 64;
+            if (b * waves < best) { best = b * waves; threads = waves * 64; }
+        }
+    }
     const int cols = threads / R;
     const bool pieces = n_tok > LA_TB;
     if (pieces && (!scratch_dev || scratch_floats < pi_op_linear_attention_scratch_floats(heads, dim, vdim, n_tok, max_segments))) { pi_set_error("pi_op_linear_attention: a pass of %d tokens needs %zu floats of scratch", n_tok, pi_op_linear_attention_scratch_floats(heads, dim, vdim, n_tok, max_segments)); return -1; }
@@ -669,7 +684,7 @@ extern "C" int pi_op_linear_attention_ex(const float * q, const float * k, const
     const double bytes = 4.0 * n_tok * heads * (2.0 * dim + 2.0 * vdim) + 8.0 * heads * dim * vdim;
     hipStream_t s = (hipStream_t) stream;
     const int nta = std::min(n_tok, PI_KT_MAXNT - 1);
-#define LA_GO(D, MODE) PI_KT_LAUNCH(PI_KT_ATT, 0, nta, bytes, k_linear_attention<D>, grid, dim3(threads), lds, s, q, k, v, stride, heads, hpg, dim, vdim, R, decay_dev, tdecay_dev, tscale_dev, t_stride, skip_dev, state_dev, rec_dev, n_tok, MODE, scratch_dev, out, out_stride, pi_abort_word())
+#define LA_GO(D, MODE) PI_KT_LAUNCH(PI_KT_ATT, 0, nta, bytes, k_linear_attention<D>, grid, dim3(threads), lds, s, q, k, v, stride, heads, hpg, dim, vdim, value_cols, R, decay_dev, tdecay_dev, tscale_dev, t_stride, skip_dev, state_dev, rec_dev, n_tok, MODE, scratch_dev, out, out_stride, pi_abort_word())
 #define LA_ANY(MODE) do { if (dpt == 8) LA_GO(8, MODE); else if (dpt == 16) LA_GO(16, MODE); else LA_GO(32, MODE); } while (0)
     if (!pieces) { LA_ANY(0); PI_CHECK_LAUNCH(); return 0; }
     LA_ANY(1);
@@ -700,10 +715,12 @@ extern "C" int pi_op_copy_f32(const float * src, float * dst, int64_t n, void * 
 // broadcast from LDS to M x RPT accumulators; every split leaves an un-normalised partial (max, sum, sum of p * c) in scratch.  (3) k_latent_combine merges the splits with
 // the sink term, normalises and applies the value up-projection.  K / V are never materialised; single tokens are spread over the chip by the splits (64 cells each),
 // prompts take splits only when a score row would not fit LDS.
-// scratch (floats): qa [n_tok][heads][rank] | pol [n_tok][heads][S][rank] | pml [n_tok][heads][S][2]
+// A cached row is [latent (rank) | rotated key part (rot values, shared by the heads; none by default)]: the folded query carries its own rotated part behind the rank values, so a score is one
+// dot product over the row's width; only the latent is summed with the probabilities.  Which cells a token sees is the mask's alone (a window of positions: pi_op_window_mask).
+// scratch (floats): qa [n_tok][heads][rank + rot] | pol [n_tok][heads][S][rank] | pml [n_tok][heads][S][2]
 #define LAT_LDS_BUDGET (128 * 1024)
 struct lat_plan { int M, RPT, cap, S; size_t lds, scratch; };
-static lat_plan latent_plan(int heads, int rank, int n_tok, int n_ctx) {
+static lat_plan latent_plan(int heads, int rank, int rot, int n_tok, int n_ctx) {
     lat_plan p;
     const bool single = n_tok <= 8;
     int best = 1;                                                     // heads per workgroup: the largest tile that leaves at most a quarter of its accumulator rows idle
@@ -716,20 +733,31 @@ static lat_plan latent_plan(int heads, int rank, int n_tok, int n_ctx) {
     p.cap = std::min(p.cap, (n_ctx + 63) / 64 * 64);
     p.S = (n_ctx + p.cap - 1) / p.cap;
     p.lds = ((size_t) p.cap * p.M + (size_t) G * p.M * rank + 8 * p.M + 8 + 256 * p.M) * 4;
-    p.scratch = (size_t) n_tok * heads * rank * (1 + p.S) + (size_t) n_tok * heads * p.S * 2;
+    p.scratch = (size_t) n_tok * heads * (rank + rot) + (size_t) n_tok * heads * rank * p.S + (size_t) n_tok * heads * p.S * 2;
     return p;
 }
 
-// grid (token tile of 4, head, 64 values of the rank): lane = one rank value, the four waves take a quarter of the head's dim each and meet in LDS
-__global__ void __launch_bounds__(256) k_latent_absorb(const float * __restrict__ q, int64_t qs, const uint16_t * __restrict__ wuk, float scale, int heads, int dim, int rank, int n_tok,
-                                                       float * __restrict__ qa, const int32_t * __restrict__ abort_w) {
+// grid (token tile of 4, head, 64 values of the rank, then 64 values of the rotated part): lane = one rank value, the four waves take a quarter of the head's dim each and meet in LDS.  A query head is
+// [dim values | rot values]; the last are turned in neighbouring pairs by the token's position (cs: the rotation table) and go behind the rank values
+__global__ void __launch_bounds__(256) k_latent_absorb(const float * __restrict__ q, int64_t qs, const uint16_t * __restrict__ wuk, float scale, int heads, int dim, int rank, int rot, const float2 * __restrict__ cs, int n_pos,
+                                                       const int32_t * __restrict__ pos, int n_tok, float * __restrict__ qa, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 5)) return;
     __shared__ float part[4][4][64];
     extern __shared__ float4 qsh[];                                    // [dim]: the head's query values of the four tokens, side by side
     const int t0 = blockIdx.x * 4, h = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r = blockIdx.z * 64 + lane;
+    const int n_rank_blocks = (rank + 63) / 64, hw = dim + rot;
+    if ((int) blockIdx.z >= n_rank_blocks) {                           // the rotated part: wave = token
+        const int d = (blockIdx.z - n_rank_blocks) * 64 + lane, t = t0 + wave;
+        if (d >= rot || t >= n_tok) return;
+        const float * qr = q + (int64_t) t * qs + (int64_t) h * hw + dim;
+        const float2 c = cs[(int64_t) min(pos[t], n_pos - 1) * (rot / 2) + (d >> 1)];
+        const float own = qr[d], other = qr[d ^ 1];
+        qa[((int64_t) t * heads + h) * (rank + rot) + rank + d] = ((d & 1) ? own * c.x + other * c.y : own * c.x - other * c.y) * scale;
+        return;
+    }
     for (int idx = threadIdx.x; idx < 4 * dim; idx += 256) {
         const int tt = idx / dim, d = idx % dim;
-        ((float *) qsh)[d * 4 + tt] = q[(int64_t) min(t0 + tt, n_tok - 1) * qs + (int64_t) h * dim + d];
+        ((float *) qsh)[d * 4 + tt] = q[(int64_t) min(t0 + tt, n_tok - 1) * qs + (int64_t) h * hw + d];
     }
     __syncthreads();
     const int dq = (dim + 3) / 4, d0 = wave * dq, d1 = min(dim, d0 + dq);
@@ -745,60 +773,58 @@ __global__ void __launch_bounds__(256) k_latent_absorb(const float * __restrict_
     for (int tt = 0; tt < 4; tt++) part[wave][tt][lane] = acc[tt];
     __syncthreads();
     const int tt = wave;                                              // wave tt writes token t0 + tt
-    if (t0 + tt < n_tok && r < rank) qa[((int64_t) (t0 + tt) * heads + h) * rank + r] = (part[0][tt][lane] + part[1][tt][lane] + part[2][tt][lane] + part[3][tt][lane]) * scale;
+    if (t0 + tt < n_tok && r < rank) qa[((int64_t) (t0 + tt) * heads + h) * (rank + rot) + r] = (part[0][tt][lane] + part[1][tt][lane] + part[2][tt][lane] + part[3][tt][lane]) * scale;
 }
 
 template <int M, int RPT>
-__global__ void __launch_bounds__(256) k_latent_scores(const float * __restrict__ qa, const float * __restrict__ cache, const uint32_t * __restrict__ mask, int heads, int rank, int n_kv_arg,
+__global__ void __launch_bounds__(256) k_latent_scores(const float * __restrict__ qa, const float * __restrict__ cache, const uint32_t * __restrict__ mask, int heads, int rank, int rot, int n_kv_arg,
                                                        int cap, int S, float * __restrict__ pol, float * __restrict__ pml, const int32_t * __restrict__ dyn, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 5)) return;
     extern __shared__ float lds[];
     const int t = blockIdx.x, h0 = blockIdx.y * M, split = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int rthreads = (rank + RPT - 1) / RPT, G = max(1, 256 / rthreads);
     float * sc = lds, * part = sc + (size_t) cap * M, * red = part + (size_t) G * M * rank, * wsc = red + 8 * M + 8;     // red: [4 waves][M] twice; wsc: [4 waves][64 cells][M]
-    __shared__ int hi_s;
+    __shared__ int hi_s, lo_s;
     const int n_kv = min(dyn ? dyn[1] : n_kv_arg, n_kv_arg);
     const int words = (n_kv_arg + 31) / 32;
     const uint32_t * mrow = mask + (int64_t) t * words;
-    const int c0 = split * cap;
+    int c0 = split * cap;
     int c1 = min(n_kv, c0 + cap);
-    if (tid == 0) hi_s = 0;
+    if (tid == 0) { hi_s = 0; lo_s = 0x7fffffff; }
     __syncthreads();
-    {   // cells past the last visible one of this token are not walked (a prompt's early tokens see little of the pass's cells)
-        int hi = 0;
-        for (int w = (c0 >> 5) + tid; w < (c1 + 31) >> 5; w += 256) { const uint32_t bits = mrow[w]; if (bits) hi = max(hi, w * 32 + 32 - __clz(bits)); }
-        if (hi) atomicMax(&hi_s, hi);
+    {   // cells past the last visible one of this token are not walked (a prompt's early tokens see little of the pass's cells), nor those ahead of the first (a window's)
+        int hi = 0, lo = 0x7fffffff;
+        for (int w = (c0 >> 5) + tid; w < (c1 + 31) >> 5; w += 256) { const uint32_t bits = mrow[w]; if (bits) { hi = max(hi, w * 32 + 32 - __clz(bits)); lo = min(lo, w * 32 + __ffs(bits) - 1); } }
+        if (hi) { atomicMax(&hi_s, hi); atomicMin(&lo_s, lo); }
     }
     __syncthreads();
-    c1 = min(c1, hi_s);
+    c1 = min(c1, hi_s); c0 = max(c0, lo_s);
+    const int W = rank + rot;                                          // a cached row
     const int nh = min(M, heads - h0);
-    const float * qat = qa + ((int64_t) t * heads + h0) * rank;
+    const float * qat = qa + ((int64_t) t * heads + h0) * W;
     float * pol_t = pol + (((int64_t) t * heads + h0) * S + split) * rank, * pml_t = pml + (((int64_t) t * heads + h0) * S + split) * 2;
-    if (c1 <= c0) {                                                   // nothing of this token lives in this split: an empty partial
-        for (int m = 0; m < nh; m++) {
-            for (int r = tid; r < rank; r += 256) pol_t[(int64_t) m * S * rank + r] = 0.0f;
-            if (tid == 0) { pml_t[(int64_t) m * S * 2] = -INFINITY; pml_t[(int64_t) m * S * 2 + 1] = 0.0f; }
-        }
+    if (c1 <= c0) {                                                   // nothing of this token lives in this split: its maximum says so, and nobody reads its sums
+        if (tid < nh) { pml_t[(int64_t) tid * S * 2] = -INFINITY; pml_t[(int64_t) tid * S * 2 + 1] = 0.0f; }
         return;
     }
     // scores: a thread per cell; a split of 64 cells (single tokens) gives every wave a quarter of the rank instead, so that all four waves stream the 64 latents
     float lmax[M];
 #pragma unroll
     for (int m = 0; m < M; m++) lmax[m] = -INFINITY;
-    if (cap == 64 && (rank & 15) == 0) {
-        const int j = c0 + lane, rq = rank >> 2, rb = wave * rq;
+    if (cap == 64 && (W & 15) == 0) {
+        const int j = c0 + lane, rq = W >> 2, rb = wave * rq;
         const bool vis = j < c1 && ((mrow[j >> 5] >> (j & 31)) & 1u);
         float a[M];
 #pragma unroll
         for (int m = 0; m < M; m++) a[m] = 0.0f;
         if (vis) {
-            const float * c = cache + (int64_t) j * rank + rb;
+            const float * c = cache + (int64_t) j * W + rb;
 #pragma unroll 8
             for (int r = 0; r < rq; r += 4) {
                 const float4 cv = *(const float4 *) (c + r);
 #pragma unroll
                 for (int m = 0; m < M; m++) {
-                    const float * qq = qat + (m < nh ? m : 0) * rank + rb + r;                    // (wave-uniform address)
+                    const float * qq = qat + (m < nh ? m : 0) * W + rb + r;                    // (wave-uniform address)
                     a[m] = fmaf(qq[0], cv.x, a[m]); a[m] = fmaf(qq[1], cv.y, a[m]); a[m] = fmaf(qq[2], cv.z, a[m]); a[m] = fmaf(qq[3], cv.w, a[m]);
                 }
             }
@@ -821,22 +847,22 @@ __global__ void __launch_bounds__(256) k_latent_scores(const float * __restrict_
 #pragma unroll
         for (int m = 0; m < M; m++) a[m] = 0.0f;
         if (vis) {
-            const float * c = cache + (int64_t) j * rank;
-            if ((rank & 3) == 0) {
+            const float * c = cache + (int64_t) j * W;
+            if ((W & 3) == 0) {
 #pragma unroll 2
-                for (int r = 0; r < rank; r += 4) {
+                for (int r = 0; r < W; r += 4) {
                     const float4 cv = *(const float4 *) (c + r);
 #pragma unroll
                     for (int m = 0; m < M; m++) {
-                        const float * qq = qat + (m < nh ? m : 0) * rank + r;                     // (wave-uniform address)
+                        const float * qq = qat + (m < nh ? m : 0) * W + r;                     // (wave-uniform address)
                         a[m] = fmaf(qq[0], cv.x, a[m]); a[m] = fmaf(qq[1], cv.y, a[m]); a[m] = fmaf(qq[2], cv.z, a[m]); a[m] = fmaf(qq[3], cv.w, a[m]);
                     }
                 }
             } else {
-                for (int r = 0; r < rank; r++) {
+                for (int r = 0; r < W; r++) {
                     const float cv = c[r];
 #pragma unroll
-                    for (int m = 0; m < M; m++) a[m] = fmaf(qat[(m < nh ? m : 0) * rank + r], cv, a[m]);
+                    for (int m = 0; m < M; m++) a[m] = fmaf(qat[(m < nh ? m : 0) * W + r], cv, a[m]);
                 }
             }
         }
@@ -877,7 +903,7 @@ __global__ void __launch_bounds__(256) k_latent_scores(const float * __restrict_
         for (int j = c0 + g; j < c1; j += G) {                          // (a masked cell has p = 0: its latent — zeros or an earlier owner's finite values — adds nothing)
             float cv[RPT];
 #pragma unroll
-            for (int i = 0; i < RPT; i++) cv[i] = r0 + i < rank ? cache[(int64_t) j * rank + r0 + i] : 0.0f;
+            for (int i = 0; i < RPT; i++) cv[i] = r0 + i < rank ? cache[(int64_t) j * W + r0 + i] : 0.0f;
             const float * pj = sc + (size_t) (j - c0) * M;
 #pragma unroll
             for (int m = 0; m < M; m++) {
@@ -909,18 +935,20 @@ __global__ void __launch_bounds__(256) k_latent_scores(const float * __restrict_
     }
 }
 
-// grid (token tile of 4, head, 16 output values): merges the splits (with the sink), normalises, applies its rows of W_uv[h]
+// grid (token tile of 4, head, 16 output values): merges the splits (with the sink if there is one), normalises, applies its rows of W_uv[h], then the head's gate if there is one
 __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict__ pol, const float * __restrict__ pml, const uint16_t * __restrict__ wuv, const float * __restrict__ sink,
-                                                        int heads, int vdim, int rank, int S, int n_tok, float * __restrict__ out, int64_t os, const int32_t * __restrict__ abort_w) {
+                                                        const float * __restrict__ gate, int64_t gs, int gate_act, int heads, int vdim, int rank, int S, int n_tok, float * __restrict__ out, int64_t os,
+                                                        const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 5)) return;
     extern __shared__ float ol[];                                     // [4][rank]
-    __shared__ float wgt[4][64 + 1];                                  // per token: weight of every split (S <= 64 at a time), [64]: 1 / denominator
+    __shared__ float wgt[4][64];                                      // per token: weight of the splits that hold something, 64 splits at a time,
+    __shared__ int num[4][64], cnt[4];                                // their numbers, how many they are
     const int t0 = blockIdx.x * 4, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int nt = min(4, n_tok - t0);
     for (int idx = tid; idx < 4 * rank; idx += 256) ol[idx] = 0.0f;
     // (the wave `tt` owns token t0 + tt's bookkeeping)
     float mstar = -INFINITY, den = 0.0f;
-    const float sk = sink[h];
+    const float sk = sink ? sink[h] : -INFINITY;
     const float * pml_t = pml + ((int64_t) (t0 + min(wave, nt - 1)) * heads + h) * S * 2;
     {
         float m = sk;
@@ -928,22 +956,25 @@ __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict
         mstar = pi_wave_max(m);
         float d = 0.0f;
         for (int s = lane; s < S; s += 64) { const float ms = pml_t[s * 2]; if (ms != -INFINITY) d += pml_t[s * 2 + 1] * expf(ms - mstar); }
-        den = pi_lanes_sum<64>(d) + expf(sk - mstar);
+        den = pi_lanes_sum<64>(d) + (sink ? expf(sk - mstar) : 0.0f);
     }
     for (int sb = 0; sb < S; sb += 64) {
         __syncthreads();
         if (wave < nt) {
             const int s = sb + lane;
             const float ms = s < S ? pml_t[s * 2] : -INFINITY;
-            wgt[wave][lane] = ms == -INFINITY ? 0.0f : expf(ms - mstar) / den;
+            const unsigned long long some = __ballot(ms != -INFINITY);
+            if (ms != -INFINITY) { const int at = __popcll(some & ((1ull << lane) - 1ull)); wgt[wave][at] = expf(ms - mstar) / den; num[wave][at] = s; }
+            if (lane == 0) cnt[wave] = __popcll(some);
         }
         __syncthreads();
         for (int idx = tid; idx < nt * rank; idx += 256) {
             const int tt = idx / rank, r = idx % rank;
-            const float * p = pol + (((int64_t) (t0 + tt) * heads + h) * S + sb) * rank + r;
+            const float * p = pol + (((int64_t) (t0 + tt) * heads + h) * S) * rank + r;
             float v = ol[idx];
+            const int n = cnt[tt];
 #pragma unroll 8
-            for (int s = 0; s < min(64, S - sb); s++) v = fmaf(wgt[tt][s], p[(int64_t) s * rank], v);                 // (an empty split: weight 0, partial written as zeros)
+            for (int s = 0; s < n; s++) v = fmaf(wgt[tt][s], p[(int64_t) num[tt][s] * rank], v);
             ol[idx] = v;
         }
     }
@@ -958,13 +989,20 @@ __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict
             for (int tt = 0; tt < 4; tt++) a[tt] = fmaf(w, ol[tt * rank + r], a[tt]);
         }
 #pragma unroll
-        for (int tt = 0; tt < 4; tt++) { const float v = pi_lanes_sum<64>(a[tt]); if (lane == 0 && tt < nt) out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v; }
+        for (int tt = 0; tt < 4; tt++) {
+            float v = pi_lanes_sum<64>(a[tt]);
+            if (lane == 0 && tt < nt) {
+                if (gate) { const float g = gate[(int64_t) (t0 + tt) * gs + h]; v *= gate_act == PI_ACT_SIGMOID ? 1.0f / (1.0f + expf(-g)) : g; }
+                out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v;
+            }
+        }
     }
 }
 
 extern "C" int pi_op_latent_attention_max_cells(int rank) { (void) rank; return 1 << 22; }       // (long contexts are cut into splits: no score row has to fit LDS whole)
-extern "C" size_t pi_op_latent_attention_scratch_floats(int heads, int rank, int n_tok, int n_ctx) {
-    return std::max(latent_plan(heads, rank, n_tok, n_ctx).scratch, latent_plan(heads, rank, std::min(n_tok, 8), n_ctx).scratch);
+extern "C" size_t pi_op_latent_attention_scratch_floats(int heads, int rank, int n_tok, int n_ctx) { return pi_op_latent_attention_rot_scratch_floats(heads, rank, 0, n_tok, n_ctx); }
+extern "C" size_t pi_op_latent_attention_rot_scratch_floats(int heads, int rank, int rot_dim, int n_tok, int n_ctx) {
+    return std::max(latent_plan(heads, rank, rot_dim, n_tok, n_ctx).scratch, latent_plan(heads, rank, rot_dim, std::min(n_tok, 8), n_ctx).scratch);
 }
 template <int M, int RPT> static int latent_reserve_one() {
     PI_CHECK_HIP(hipFuncSetAttribute((const void *) k_latent_scores<M, RPT>, hipFuncAttributeMaxDynamicSharedMemorySize, LAT_LDS_BUDGET + 4096));
@@ -980,39 +1018,53 @@ extern "C" int pi_op_latent_attention_reserve(void) {
     return 0;
 }
 template <int M, int RPT>
-static void latent_scores_launch(const lat_plan & p, dim3 grid, hipStream_t s, double bytes, int nta, const float * qa, const float * cache, const uint32_t * mask, int heads, int rank, int n_kv,
+static void latent_scores_launch(const lat_plan & p, dim3 grid, hipStream_t s, double bytes, int nta, const float * qa, const float * cache, const uint32_t * mask, int heads, int rank, int rot, int n_kv,
                                  float * pol, float * pml, const int32_t * dyn) {
-    PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, bytes, (k_latent_scores<M, RPT>), grid, dim3(256), p.lds, s, qa, cache, mask, heads, rank, n_kv, p.cap, p.S, pol, pml, dyn, pi_abort_word());
+    PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, bytes, (k_latent_scores<M, RPT>), grid, dim3(256), p.lds, s, qa, cache, mask, heads, rank, rot, n_kv, p.cap, p.S, pol, pml, dyn, pi_abort_word());
 }
 extern "C" int pi_op_latent_attention(const float * q, int64_t q_stride, const float * cache, const uint32_t * mask, const pi_weight * wuk, const pi_weight * wuv, const float * sink_dev,
                                       float scale, int heads, int dim, int vdim, int rank, int n_tok, int n_kv, float * scratch_dev, size_t scratch_floats, float * out, int64_t out_stride,
                                       const int32_t * dyn_dev, void * stream) {
+    if (!sink_dev) { pi_set_error("pi_op_latent_attention: the sink is required"); return -1; }
+    return pi_op_latent_attention_rot(q, q_stride, cache, mask, wuk, wuv, sink_dev, nullptr, 0, PI_ACT_NONE, scale, heads, dim, 0, vdim, rank, nullptr, nullptr, n_tok, n_kv, scratch_dev, scratch_floats, out, out_stride, dyn_dev, stream);
+}
+extern "C" int pi_op_latent_attention_rot(const float * q, int64_t q_stride, const float * cache, const uint32_t * mask, const pi_weight * wuk, const pi_weight * wuv, const float * sink_dev, const float * gate_dev,
+                                          int64_t gate_stride, int gate_act, float scale, int heads, int dim, int rot, int vdim, int rank, const void * rotary_table, const int32_t * pos_dev, int n_tok, int n_kv,
+                                          float * scratch_dev, size_t scratch_floats, float * out, int64_t out_stride, const int32_t * dyn_dev, void * stream) {
     if (n_tok <= 0) return 0;
+    const float2 * cs = nullptr; int n_pos = 0, half = 0;
+    if (rot < 0 || (rot & 1)) { pi_set_error("pi_op_latent_attention: %d rotated dimensions (an even number)", rot); return -1; }
+    if (rot > 0) {
+        pi_rotary_table_view(rotary_table, &cs, &n_pos, &half);
+        if (!cs || half != rot / 2 || !pos_dev) { pi_set_error("pi_op_latent_attention: a rotation table over the %d rotated dimensions and the tokens' positions are required", rot); return -1; }
+    }
+    if (gate_dev && gate_act != PI_ACT_NONE && gate_act != PI_ACT_SIGMOID) { pi_set_error("pi_op_latent_attention: gate activation %d is unknown", gate_act); return -1; }
+    if (q_stride < (int64_t) heads * (dim + rot)) { pi_set_error("pi_op_latent_attention: query rows of %lld floats hold no %d heads of %d + %d values", (long long) q_stride, heads, dim, rot); return -1; }
     if (!wuk || !wuv || wuk->type != PI_BF16 || wuv->type != PI_BF16 || wuk->ne0 != rank || wuv->ne0 != rank || wuk->ne1 != (int64_t) heads * dim || wuv->ne1 != (int64_t) heads * vdim) {
         pi_set_error("pi_op_latent_attention: the up-projections must be bfloat16 [heads * dim][rank] and [heads * vdim][rank]"); return -1;
     }
     if (rank > 1024) { pi_set_error("pi_op_latent_attention: latent width %d above 1024", rank); return -1; }
-    const lat_plan p = latent_plan(heads, rank, n_tok, n_kv);
+    const lat_plan p = latent_plan(heads, rank, rot, n_tok, n_kv);
     if (p.scratch > scratch_floats) { pi_set_error("pi_op_latent_attention: %zu floats of scratch needed, %zu given", p.scratch, scratch_floats); return -1; }
     if (p.lds > LAT_LDS_BUDGET + 4096 || (size_t) 4 * rank * 4 > 64 * 1024) { pi_set_error("pi_op_latent_attention: LDS plan does not fit"); return -1; }
     if (pi_op_latent_attention_reserve() != 0) return -1;
     hipStream_t s = (hipStream_t) stream;
-    float * qa = scratch_dev, * pol = qa + (size_t) n_tok * heads * rank, * pml = pol + (size_t) n_tok * heads * p.S * rank;
+    float * qa = scratch_dev, * pol = qa + (size_t) n_tok * heads * (rank + rot), * pml = pol + (size_t) n_tok * heads * p.S * rank;
     const int nta = std::min(n_tok, PI_KT_MAXNT - 1);
     const int acct = pi_account_n_kv() > 0 ? pi_account_n_kv() : n_kv;
-    PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, 2.0 * rank * heads * dim + 4.0 * n_tok * heads * (dim + rank), k_latent_absorb, dim3((unsigned) ((n_tok + 3) / 4), (unsigned) heads, (unsigned) ((rank + 63) / 64)), dim3(256), (size_t) 16 * dim, s,
-                 q, q_stride, (const uint16_t *) wuk->p0, scale, heads, dim, rank, n_tok, qa, pi_abort_word());
+    PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, 2.0 * rank * heads * dim + 4.0 * n_tok * heads * (dim + rank + 2.0 * rot), k_latent_absorb, dim3((unsigned) ((n_tok + 3) / 4), (unsigned) heads, (unsigned) ((rank + 63) / 64 + (rot + 63) / 64)), dim3(256), (size_t) 16 * dim, s,
+                 q, q_stride, (const uint16_t *) wuk->p0, scale, heads, dim, rank, rot, cs, n_pos, pos_dev, n_tok, qa, pi_abort_word());
     PI_CHECK_LAUNCH();
     const dim3 grid((unsigned) n_tok, (unsigned) ((heads + p.M - 1) / p.M), (unsigned) p.S);
-    const double bytes = 4.0 * acct * rank + 4.0 * n_tok * heads * rank * (1.0 + p.S);
-#define LAT_GO(M) do { if (p.RPT == 1) latent_scores_launch<M, 1>(p, grid, s, bytes, nta, qa, cache, mask, heads, rank, n_kv, pol, pml, dyn_dev); \
-                       else if (p.RPT == 2) latent_scores_launch<M, 2>(p, grid, s, bytes, nta, qa, cache, mask, heads, rank, n_kv, pol, pml, dyn_dev); \
-                       else latent_scores_launch<M, 4>(p, grid, s, bytes, nta, qa, cache, mask, heads, rank, n_kv, pol, pml, dyn_dev); } while (0)
+    const double bytes = 4.0 * acct * (rank + rot) + 4.0 * n_tok * heads * (rank + rot + (double) rank * p.S);
+#define LAT_GO(M) do { if (p.RPT == 1) latent_scores_launch<M, 1>(p, grid, s, bytes, nta, qa, cache, mask, heads, rank, rot, n_kv, pol, pml, dyn_dev); \
+                       else if (p.RPT == 2) latent_scores_launch<M, 2>(p, grid, s, bytes, nta, qa, cache, mask, heads, rank, rot, n_kv, pol, pml, dyn_dev); \
+                       else latent_scores_launch<M, 4>(p, grid, s, bytes, nta, qa, cache, mask, heads, rank, rot, n_kv, pol, pml, dyn_dev); } while (0)
     switch (p.M) { case 16: LAT_GO(16); break; case 8: LAT_GO(8); break; case 4: LAT_GO(4); break; case 2: LAT_GO(2); break; default: LAT_GO(1); }
 #undef LAT_GO
     PI_CHECK_LAUNCH();
     PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, 2.0 * rank * heads * vdim + 4.0 * n_tok * heads * (rank * p.S + vdim), k_latent_combine, dim3((unsigned) ((n_tok + 3) / 4), (unsigned) heads, (unsigned) ((vdim + 15) / 16)), dim3(256), (size_t) 16 * rank, s,
-                 pol, pml, (const uint16_t *) wuv->p0, sink_dev, heads, vdim, rank, p.S, n_tok, out, out_stride, pi_abort_word());
+                 pol, pml, (const uint16_t *) wuv->p0, sink_dev, gate_dev, gate_stride, gate_act, heads, vdim, rank, p.S, n_tok, out, out_stride, pi_abort_word());
     PI_CHECK_LAUNCH(); return 0;
 }
 

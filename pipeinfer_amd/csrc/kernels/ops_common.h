@@ -46,6 +46,7 @@ int pi_account_n_kv();                                       // > 0: the cells a
 // compute units the launching context's stream may use (pipeinfer_context_set_cu_range -> hipExtStreamCreateWithCUMask; 256 without a mask): what "one round of workgroups" means
 int pi_cu_count();
 const pi_tables & pi_get_tables();
+void pi_rotary_table_view(const void * table, const float2 ** cs, int * n_pos, int * half);      // a rotation table's device rows [n_pos][half] of (cos, sin) (nothing for a null table)
 
 #define PI_CHECK_HIP(expr)                                                                   \
     do {                                                                                     \

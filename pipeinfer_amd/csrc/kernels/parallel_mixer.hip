@@ -56,6 +56,11 @@ static __device__ __forceinline__ void pm_pool_block(float * __restrict__ kc, fl
 
 // ---- rotation table: cos / sin of p * base^(-2i / dims), angles formed in double on the host ------------------------------------------------------------
 struct pi_rotary_table { float2 * cs; int n_pos, half; };
+static void * rotary_upload(pi_rotary_table * t, const std::vector<float2> & h) {
+    t->cs = (float2 *) pi_malloc(h.size() * sizeof(float2));
+    if (!t->cs || pi_memcpy_h2d(t->cs, h.data(), h.size() * sizeof(float2), nullptr) != 0 || pi_stream_sync(nullptr) != 0) { pi_free(t->cs); delete t; return nullptr; }
+    return t;
+}
 extern "C" void * pi_rotary_table_create(int n_pos, int dims, float base) { return pi_rotary_table_create_scaled(n_pos, dims, base, 1.0f, 1.0f, 1.0f, 0); }
 // original > 0: long wavelengths are stretched — an angle step whose wavelength 2 pi / f exceeds original / low is divided by `factor`, one below original / high stays, between the two they blend
 extern "C" void * pi_rotary_table_create_scaled(int n_pos, int dims, float base, float factor, float low, float high, int original) {
@@ -73,9 +78,28 @@ extern "C" void * pi_rotary_table_create_scaled(int n_pos, int dims, float base,
         }
         for (int p = 0; p < n_pos; p++) { const double a = (double) p * f; h[(size_t) p * t->half + i] = make_float2((float) std::cos(a), (float) std::sin(a)); }
     }
-    t->cs = (float2 *) pi_malloc(h.size() * sizeof(float2));
-    if (!t->cs || pi_memcpy_h2d(t->cs, h.data(), h.size() * sizeof(float2), nullptr) != 0 || pi_stream_sync(nullptr) != 0) { pi_free(t->cs); delete t; return nullptr; }
-    return t;
+    return rotary_upload(t, h);
+}
+// the other way to stretch: along a ramp over the pair index i between the pairs that make `fast` and `slow` turns over `original` positions (0 below: the step stays, 1 above: it is divided by `factor`),
+// and every cos and sin times 0.1 ln(factor) + 1
+extern "C" void * pi_rotary_table_create_ramp(int n_pos, int dims, float base, float factor, int original, float fast, float slow) {
+    if (n_pos < 1 || dims < 0 || (dims & 1)) { pi_set_error("pi_rotary_table_create: %d positions, %d rotated dimensions (an even number)", n_pos, dims); return nullptr; }
+    if (!(factor > 0.0f) || original < 1 || !(fast > 0.0f) || !(slow > 0.0f) || !(base > 0.0f) || base == 1.0f) { pi_set_error("pi_rotary_table_create_ramp: positive factor, original, fast, slow and a base other than 1 are required"); return nullptr; }
+    pi_rotary_table * t = new pi_rotary_table{ nullptr, n_pos, dims / 2 };
+    if (t->half == 0) return t;
+    auto index_of = [&](double turns) { return dims * std::log((double) original / (2.0 * M_PI * turns)) / (2.0 * std::log((double) base)); };
+    const double lo = std::max(std::floor(index_of(fast)), 0.0), hi = std::min(std::ceil(index_of(slow)), (double) dims - 1.0), span = std::max(hi - lo, 0.001);
+    const double amp = 0.1 * std::log((double) factor) + 1.0;
+    std::vector<float2> h((size_t) n_pos * t->half);
+    for (int i = 0; i < t->half; i++) {
+        const double f0 = std::pow((double) base, -2.0 * i / dims), r = std::min(std::max((i - lo) / span, 0.0), 1.0), f = f0 / factor * r + f0 * (1.0 - r);
+        for (int p = 0; p < n_pos; p++) { const double a = (double) p * f; h[(size_t) p * t->half + i] = make_float2((float) (amp * std::cos(a)), (float) (amp * std::sin(a))); }
+    }
+    return rotary_upload(t, h);
+}
+void pi_rotary_table_view(const void * table, const float2 ** cs, int * n_pos, int * half) {
+    const pi_rotary_table * t = (const pi_rotary_table *) table;
+    *cs = t ? t->cs : nullptr; *n_pos = t ? t->n_pos : 0; *half = t ? t->half : 0;
 }
 extern "C" int pi_rotary_table_positions(const void * table) { return table ? ((const pi_rotary_table *) table)->n_pos : 0; }
 extern "C" void pi_rotary_table_free(void * table) { pi_rotary_table * t = (pi_rotary_table *) table; if (t) { pi_free(t->cs); delete t; } }
@@ -138,14 +162,14 @@ extern "C" int pi_op_qkv_prepare(const float * q, const float * k, const float *
 // the same with the order and the pairing as parameters.  norm_first: R(.) * w, then the rotation (as above), else the rotation first and R(.) * w over the rotated head; w may be absent (1);
 // pairing PI_PAIR_HALVES: dimension i with i + dims / 2, PI_PAIR_NEIGHBOURS: 2i with 2i + 1 (angle number i either way); v_norm = 0: value heads go to their cell as they are
 __global__ void __launch_bounds__(64) k_qkv_prepare_any(const float * __restrict__ q, const float * __restrict__ k, const float * __restrict__ v, int64_t stride, const float * __restrict__ qw,
-                                                        const float * __restrict__ kw, float eps, int H, int G, int D, int V, const float2 * __restrict__ rot, int half, int n_pos, int norm_first, int pairing, int v_norm,
+                                                        const float * __restrict__ kw, float eps, int H, int G, int D, int V, const float2 * __restrict__ rot, int half, int n_pos, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every,
                                                         const int32_t * __restrict__ pos, float * __restrict__ q_out, int64_t qos, float * __restrict__ kc, float * __restrict__ vc,
                                                         int32_t * __restrict__ cell_pos, const int32_t * __restrict__ dyn, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w)) return;
     const int t = blockIdx.x, slot = blockIdx.y, lane = threadIdx.x;
     const int cell = pi_cell_of(dyn, 0, t);
     const int p = pos[t];
-    if (slot == 0 && lane == 0) cell_pos[cell] = p;
+    if (k && slot == 0 && lane == 0) cell_pos[cell] = p;                // (queries alone: the cells belong to the layer whose keys are read)
     if (slot >= H + G) {
         const int g = slot - H - G;
         const float * src = v + (int64_t) t * stride + (int64_t) g * V;
@@ -164,6 +188,7 @@ __global__ void __launch_bounds__(64) k_qkv_prepare_any(const float * __restrict
     const float * src = (is_q ? q : k) + (int64_t) t * stride + (int64_t) h * D;
     const float * w = is_q ? qw : kw;
     float * dst = is_q ? q_out + (int64_t) t * qos + (int64_t) h * D : kc + ((int64_t) cell * G + h) * D;
+    const float temp = is_q && temp_every > 0 ? fmaf(temp_coef, logf((float) ((p + 1) / temp_every + 1)), 1.0f) : 1.0f;       // query temperature: grows with the logarithm of the position's block
     const bool none = norm_first == PI_QK_NORM_NONE;
     norm_first = norm_first == PI_QK_NORM_FIRST;
     float inv1 = 1.0f;
@@ -185,25 +210,32 @@ __global__ void __launch_bounds__(64) k_qkv_prepare_any(const float * __restrict
         }
         return y;
     };
-    if (norm_first || none) { for (int i = lane; i < D; i += 64) dst[i] = turned(i); return; }
+    if (norm_first || none) { for (int i = lane; i < D; i += 64) dst[i] = turned(i) * temp; return; }
     float ss = 0.0f;
     for (int i = lane; i < D; i += 64) { const float y = turned(i); ss = fmaf(y, y, ss); }
     const float inv = 1.0f / sqrtf(pi_lanes_sum<64>(ss) / (float) D + eps);
-    for (int i = lane; i < D; i += 64) dst[i] = turned(i) * inv * (w ? w[i] : 1.0f);
+    for (int i = lane; i < D; i += 64) dst[i] = turned(i) * inv * (w ? w[i] : 1.0f) * temp;
 }
 extern "C" int pi_op_qkv_prepare_ex(const float * q, const float * k, const float * v, int64_t stride, const float * q_norm_w, const float * k_norm_w, float eps, int heads, int kv_heads, int dim, int vdim,
                                     const void * rotary_table, int norm_first, int pairing, int v_norm, const int32_t * pos_dev, int n_tok, float * q_out, int64_t q_out_stride, float * k_cache, float * v_cache,
                                     int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream) {
+    if (n_tok > 0 && (!k || !v)) { pi_set_error("pi_op_qkv_prepare: keys and values are required"); return -1; }
+    return pi_op_qkv_prepare_temp(q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, dim, vdim, rotary_table, norm_first, pairing, v_norm, 0.0f, 0, pos_dev, n_tok, q_out, q_out_stride, k_cache, v_cache, cell_pos_dev, dyn_dev, stream);
+}
+extern "C" int pi_op_qkv_prepare_temp(const float * q, const float * k, const float * v, int64_t stride, const float * q_norm_w, const float * k_norm_w, float eps, int heads, int kv_heads, int dim, int vdim,
+                                      const void * rotary_table, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every, const int32_t * pos_dev, int n_tok, float * q_out, int64_t q_out_stride,
+                                      float * k_cache, float * v_cache, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream) {
     if (n_tok <= 0) return 0;
     const pi_rotary_table * rt = (const pi_rotary_table *) rotary_table;
     if (!rt || 2 * rt->half > dim) { pi_set_error("pi_op_qkv_prepare: a rotation table over at most %d dimensions is required", dim); return -1; }
     if (heads < 1 || kv_heads < 1 || heads % kv_heads) { pi_set_error("pi_op_qkv_prepare: %d query heads do not divide over %d key / value heads", heads, kv_heads); return -1; }
-    if (!dyn_dev || !cell_pos_dev) { pi_set_error("pi_op_qkv_prepare: the pass's cell table and the cells' position array are required"); return -1; }
+    if (!k != !v || temp_every < 0) { pi_set_error("pi_op_qkv_prepare: keys and values come together, the temperature's block of positions is not negative"); return -1; }
+    if (!dyn_dev || (k && !cell_pos_dev)) { pi_set_error("pi_op_qkv_prepare: the pass's cell table and the cells' position array are required"); return -1; }
     if (pairing != PI_PAIR_HALVES && pairing != PI_PAIR_NEIGHBOURS) { pi_set_error("pi_op_qkv_prepare: pairing %d is unknown", pairing); return -1; }
     if (norm_first < 0 || norm_first > PI_QK_NORM_NONE) { pi_set_error("pi_op_qkv_prepare: norm order %d is unknown", norm_first); return -1; }
     if (norm_first == PI_QK_NORM_FIRST && (!q_norm_w || !k_norm_w)) { pi_set_error("pi_op_qkv_prepare: norm weights are required"); return -1; }
-    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 8.0 * n_tok * ((double) heads * dim + (double) kv_heads * (dim + vdim)), k_qkv_prepare_any, dim3((unsigned) n_tok, (unsigned) (heads + 2 * kv_heads)), dim3(64), 0, (hipStream_t) stream,
-                 q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, dim, vdim, rt->cs, rt->half, rt->n_pos, norm_first, pairing, v_norm, pos_dev, q_out, q_out_stride, k_cache, v_cache, cell_pos_dev, dyn_dev, pi_abort_word());
+    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 8.0 * n_tok * ((double) heads * dim + (double) kv_heads * (dim + vdim)), k_qkv_prepare_any, dim3((unsigned) n_tok, (unsigned) (heads + (k ? 2 * kv_heads : 0))), dim3(64), 0, (hipStream_t) stream,
+                 q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, dim, vdim, rt->cs, rt->half, rt->n_pos, norm_first, pairing, v_norm, temp_coef, temp_every, pos_dev, q_out, q_out_stride, k_cache, v_cache, cell_pos_dev, dyn_dev, pi_abort_word());
     PI_CHECK_LAUNCH(); return 0;
 }
 

@@ -196,3 +196,16 @@ def _declare(lib):
     lib.pi_op_moe_experts_glu.argtypes = [vp, vp, i32, i32, i32, f32, vp, i64, vp, vp, i32, i32, i32, vp, vp, i64, vp]
     lib.pi_op_moe_experts_grouped_glu.argtypes = [vp, vp, i32, i32, i32, f32, vp, i64, vp, vp, i32, i32, vp, vp, vp, vp, i64, vp]
     lib.pi_op_glu_mul_ex.argtypes = [vp, i64, i32, i32, f32, i64, i32, vp, i64, vp]
+    # several residual streams, normalised matrix memories, latent attention with a rotated part and a window, query temperatures
+    lib.pi_op_dense_bias.argtypes = [vp, vp, vp, i64, i32, vp, i64, i32, i64, i32, i32, vp]
+    lib.pi_op_hyper_step.argtypes = [vp, i64, i64, i32, vp, i64, vp, vp, vp, vp, f32, i32, i32, vp, vp, i64, vp]
+    lib.pi_op_memory_gates.argtypes = [vp, vp, i64, vp, vp, f32, i32, vp, vp, i32, vp, vp, vp, vp]
+    lib.pi_op_linear_attention_keysum.argtypes = [vp, vp, vp, i64, i32, i32, i32, i32, i32, vp, vp, vp, i64, vp, vp, vp, i32, i32, vp, sz, vp, i64, vp]
+    lib.pi_op_memory_norm.argtypes = [vp, i64, vp, f32, f32, i32, i32, f32, vp, vp, i64, i32, i32, vp, i64, vp]
+    lib.pi_rotary_table_create_ramp.restype = vp
+    lib.pi_rotary_table_create_ramp.argtypes = [i32, i32, f32, f32, i32, f32, f32]
+    lib.pi_op_qkv_prepare_temp.argtypes = [vp, vp, vp, i64, vp, vp, f32, i32, i32, i32, i32, vp, i32, i32, i32, f32, i32, vp, i32, vp, i64, vp, vp, vp, vp, vp]
+    lib.pi_op_window_mask.argtypes = [vp, vp, vp, i32, i32, i32, vp, vp, vp]
+    lib.pi_op_latent_prepare.argtypes = [vp, i64, i32, vp, i32, vp, i32, vp, f32, vp, i32, vp, i64, vp, vp, vp]
+    lib.pi_op_latent_attention_rot.argtypes = [vp, i64, vp, vp, vp, vp, vp, vp, i64, i32, f32, i32, i32, i32, i32, i32, vp, vp, i32, i32, vp, sz, vp, i64, vp, vp]
+    lib.pi_op_latent_attention_rot_scratch_floats.argtypes = [i32, i32, i32, i32, i32]; lib.pi_op_latent_attention_rot_scratch_floats.restype = sz
