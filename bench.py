@@ -499,7 +499,13 @@ def main():
     ap.add_argument("--compare-window", nargs="?", const="w1024,w2048,w4096", default=None, metavar="SIZES",
                     help="instead of the default workload: the same measurements for the Rarevik design (one tanh norm per layer, sliding-window attention with pooled far blocks, clipped routed experts) "
                          "beside the Vikarax design at equal sizes; one JSON line per size")
+    ap.add_argument("--compare-streams", nargs="?", const="w1024,w2048,w4096", default=None, metavar="SIZES",
+                    help="instead of the default workload: the same measurements for the Rerizen design (residual streams, matrix memories, windowed latent attention behind a query latent) beside the Fasovik "
+                         "design at equal sizes; one JSON line per size")
     args = ap.parse_args()
+    if args.compare_streams:
+        from pipeinfer_amd.tools import hybrid_bench
+        return hybrid_bench.main_streams(args.compare_streams.split(","), args.cache)
     if args.compare_window:
         from pipeinfer_amd.tools import hybrid_bench
         return hybrid_bench.main_window(args.compare_window.split(","), args.cache)

@@ -606,24 +606,28 @@ __global__ void __launch_bounds__(256) k_linear_state_scan(int heads, int dim, i
     if (nsub == 0 || word < 0) return;
     const int h = blockIdx.x, slot = word & ~LA_FRESH;
     const int64_t per = (int64_t) dim * vdim, idx = (int64_t) blockIdx.y * 256 + threadIdx.x;
-    if (idx >= per) return;
+    const bool in = idx < per;
+    __shared__ float lps[8];                                           // per-token decays: their products over eight pieces, a thread per token (LA_TB = 32 lanes meet per piece)
     float lp = 1.0f;                                                   // lambda^LA_TB: every piece but a run's last has LA_TB tokens
     if (!tdecay) for (int i = 0; i < LA_TB; i++) lp *= decay[h];
-    float run = (word & LA_FRESH) ? 0.0f : state[((int64_t) slot * heads + h) * per + idx];
+    float run = !in || (word & LA_FRESH) ? 0.0f : state[((int64_t) slot * heads + h) * per + idx];
     for (int p0 = 0; p0 < nsub; p0 += 8) {                             // eight pieces at a time: their loads are in flight together, then the chain runs on registers
         float lpart[8];
 #pragma unroll
-        for (int i = 0; i < 8; i++) lpart[i] = p0 + i < nsub - 1 ? scratch[((int64_t) (sub0 + p0 + i) * heads + h) * per + idx] : 0.0f;
+        for (int i = 0; i < 8; i++) lpart[i] = in && p0 + i < nsub - 1 ? scratch[((int64_t) (sub0 + p0 + i) * heads + h) * per + idx] : 0.0f;
+        if (tdecay) {
+            const int pi = threadIdx.x / LA_TB;                        // (256 threads: eight pieces; only whole pieces are multiplied out)
+            float d = p0 + pi < nsub - 1 ? tdecay[(int64_t) (tfirst + (p0 + pi) * LA_TB + threadIdx.x % LA_TB) * tds + h] : 1.0f;
+            for (int o = LA_TB >> 1; o > 0; o >>= 1) d *= __shfl_xor(d, o, PI_WAVE);
+            __syncthreads();                                           // (the previous eight are no longer read)
+            if (threadIdx.x % LA_TB == 0) lps[pi] = d;
+            __syncthreads();
+        }
 #pragma unroll
         for (int i = 0; i < 8; i++)
-            if (p0 + i < nsub) {
+            if (in && p0 + i < nsub) {
                 scratch[((int64_t) (sub0 + p0 + i) * heads + h) * per + idx] = run;
-                if (tdecay && p0 + i < nsub - 1) {                     // per-token decays: the product over the piece's tokens
-                    lp = 1.0f;
-                    const float * td = tdecay + (int64_t) (tfirst + (p0 + i) * LA_TB) * tds + h;
-                    for (int j = 0; j < LA_TB; j++) lp *= td[(int64_t) j * tds];
-                }
-                run = fmaf(lp, run, lpart[i]);
+                run = fmaf(tdecay ? lps[i] : lp, run, lpart[i]);
             }
     }
 }
@@ -943,9 +947,15 @@ __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict
     extern __shared__ float ol[];                                     // [4][rank]
     __shared__ float wgt[4][64];                                      // per token: weight of the splits that hold something, 64 splits at a time,
     __shared__ int num[4][64], cnt[4];                                // their numbers, how many they are
+    __shared__ float gsh[4];                                          // per token: the head's gate
     const int t0 = blockIdx.x * 4, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int nt = min(4, n_tok - t0);
     for (int idx = tid; idx < 4 * rank; idx += 256) ol[idx] = 0.0f;
+    if (tid < 4) {
+        float g = 1.0f;
+        if (gate && tid < nt) { g = gate[(int64_t) (t0 + tid) * gs + h]; if (gate_act == PI_ACT_SIGMOID) g = 1.0f / (1.0f + expf(-g)); }
+        gsh[tid] = g;
+    }
     // (the wave `tt` owns token t0 + tt's bookkeeping)
     float mstar = -INFINITY, den = 0.0f;
     const float sk = sink ? sink[h] : -INFINITY;
@@ -990,11 +1000,8 @@ __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict
         }
 #pragma unroll
         for (int tt = 0; tt < 4; tt++) {
-            float v = pi_lanes_sum<64>(a[tt]);
-            if (lane == 0 && tt < nt) {
-                if (gate) { const float g = gate[(int64_t) (t0 + tt) * gs + h]; v *= gate_act == PI_ACT_SIGMOID ? 1.0f / (1.0f + expf(-g)) : g; }
-                out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v;
-            }
+            const float v = pi_lanes_sum<64>(a[tt]);
+            if (lane == 0 && tt < nt) out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v * gsh[tt];
         }
     }
 }

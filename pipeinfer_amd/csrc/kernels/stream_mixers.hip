@@ -2,7 +2,7 @@
 // with a rotated key part and a sliding window.  Everything here is fp32 in both precisions of the engine: streams, norms, gates and their running maximum, angles.
 //
 //   k_hyper_step       x_t <- sum_s mix[s][t] x_s + out[t] y over the streams of a token, the next sublayer's input sum_s in[s] x_s and its RMS norm in one pass over the row
-//   k_memory_gates     capped log gates and their running maximum (a max-plus scan over the tokens of a sequence, 64 at a time), as factors the linear recurrence takes per token
+//   k_memory_gates     capped log gates and their running maximum (a max-plus scan over the tokens of a sequence), as factors the linear recurrence takes per token
 //   k_memory_norm      the memory's output divided by its normaliser, per-head RMS norm, weight, output gate
 //   k_window_mask      the pass's mask rows restricted to a window of positions
 //   k_latent_prepare   both latents of a token normed, the shared key part rotated; the key / value row goes to the token's cache cell
@@ -111,47 +111,51 @@ extern "C" int pi_op_hyper_step(const float * x_in, int64_t token_stride, int64_
 }
 
 // ---- gates of the matrix memory -----------------------------------------------------------------------------------------------------------------------
-// one wave per head walks the pass 64 tokens at a time.  m' = max(f + m, i) is affine in the max-plus sense: token t is the pair (f, i), two neighbours combine to (f1 + f2, max(i1 + f2, i2)), and a
-// sequence's first token takes the m it starts from into its i and blocks what lies before it with f = -infinity, so the runs of a pass need no loop of their own.  The factors are formed from the very m
-// that is handed on, whatever the scan's order rounded it to.
-__global__ void __launch_bounds__(64) k_memory_gates(const float * __restrict__ ri, const float * __restrict__ rf, int64_t stride, const float * __restrict__ bi, const float * __restrict__ bf, float cap, int heads,
-                                                     float * m_state, const int32_t * __restrict__ rec, int n_tok, float * __restrict__ forget, float * __restrict__ put, float * __restrict__ flo,
-                                                     const int32_t * __restrict__ abort_w) {
+// one workgroup per head walks the pass 64 tokens per wave at a time.  m' = max(f + m, i) is affine in the max-plus sense: token t is the pair (f, i), two neighbours combine to (f1 + f2, max(i1 + f2, i2)).
+// A sequence's first token takes the m it starts from into its i and blocks what lies before it with f = -infinity, so the runs of a pass need no loop of their own.  Every wave scans its tokens, the waves'
+// totals are chained through LDS.  The factors are formed from the very m that is handed on, whatever the scan's order rounded it to.
+__global__ void __launch_bounds__(1024) k_memory_gates(const float * __restrict__ ri, const float * __restrict__ rf, int64_t stride, const float * __restrict__ bi, const float * __restrict__ bf, float cap, int heads,
+                                                       float * m_state, const int32_t * __restrict__ rec, int n_tok, float * __restrict__ forget, float * __restrict__ put, float * __restrict__ flo,
+                                                       const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w)) return;
-    const int h = blockIdx.x, lane = threadIdx.x;
+    __shared__ float tot[16][2];
+    const int h = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
     const float bih = bi[h], bfh = bf[h];
-    float m_last = 0.0f;                                               // m behind the previous 64 tokens
-    for (int t0 = 0; t0 < n_tok; t0 += 64) {
-        const int t = t0 + lane;
+    float m_base = 0.0f;                                               // m ahead of this round's tokens (a pass's first token starts a run: it does not look at it)
+    for (int t0 = 0; t0 < n_tok; t0 += blockDim.x) {
+        const int t = t0 + threadIdx.x;
         const bool ok = t < n_tok;
         const int word = ok ? rec[t] : -1, slot = word & ~SM_FRESH;
         const bool first = ok && (t == 0 || (rec[t - 1] & ~SM_FRESH) != slot), last = ok && (t + 1 == n_tok || (rec[t + 1] & ~SM_FRESH) != slot);
         const float i = ok ? cap * tanhf((ri[(int64_t) t * stride + h] + bih) / cap) : -INFINITY;
         const float a = ok ? cap * tanhf((rf[(int64_t) t * stride + h] + bfh) / cap) : 0.0f;
-        const float f = fminf(a, 0.0f) - log1pf(expf(-fabsf(a)));     // log sigmoid(a)
-        const float m_in = first ? ((word & SM_FRESH) ? 0.0f : m_state[(int64_t) slot * heads + h]) : m_last;       // (used by a run's first token and by lane 0)
-        float F = first ? -INFINITY : ok ? f : 0.0f, M = first || lane == 0 ? fmaxf(f + m_in, i) : i;
-        if (!ok) M = -INFINITY;
-        if (lane == 0) F = -INFINITY;                                  // (nothing lies before it: m_last is in its M)
+        const float f = ok ? fminf(a, 0.0f) - log1pf(expf(-fabsf(a))) : 0.0f;          // log sigmoid(a)
+        const float m_in = first && !(word & SM_FRESH) ? m_state[(int64_t) slot * heads + h] : 0.0f;
+        float F = first ? -INFINITY : f, M = first ? fmaxf(f + m_in, i) : i;
         for (int d = 1; d < 64; d <<= 1) {
             const float Fp = __shfl_up(F, d, 64), Mp = __shfl_up(M, d, 64);
             if (lane >= d) { M = fmaxf(Mp + F, M); F = Fp + F; }
         }
-        const float prev = __shfl_up(M, 1, 64);
-        const float m_prev = first || lane == 0 ? m_in : prev;
+        if (t0) __syncthreads();                                       // (the previous round's totals are no longer read)
+        if (lane == 63) { tot[wave][0] = F; tot[wave][1] = M; }
+        __syncthreads();
+        float m_wave = m_base, m_end = m_base;
+        for (int w = 0; w < waves; w++) { if (w == wave) m_wave = m_end; m_end = fmaxf(m_end + tot[w][0], tot[w][1]); }
+        const float m = fmaxf(m_wave + F, M);                          // behind this token
+        const float prev = __shfl_up(m, 1, 64), m_prev = first ? m_in : lane == 0 ? m_wave : prev;
         if (ok) {
             const int64_t o = (int64_t) t * heads + h;
-            forget[o] = expf(f + m_prev - M); put[o] = expf(i - M); flo[o] = expf(-M);
-            if (last) m_state[(int64_t) slot * heads + h] = M;
+            forget[o] = expf(f + m_prev - m); put[o] = expf(i - m); flo[o] = expf(-m);
+            if (last) m_state[(int64_t) slot * heads + h] = m;
         }
-        m_last = __shfl(M, 63, 64);
+        m_base = m_end;
     }
 }
 extern "C" int pi_op_memory_gates(const float * raw_i, const float * raw_f, int64_t stride, const float * bias_i_dev, const float * bias_f_dev, float cap, int heads, float * m_state_dev, const int32_t * rec_dev, int n_tok,
                                   float * forget_dev, float * put_dev, float * floor_dev, void * stream) {
     if (n_tok <= 0) return 0;
     if (heads < 1 || !(cap > 0.0f) || !raw_i || !raw_f || !bias_i_dev || !bias_f_dev || !m_state_dev || !rec_dev) { pi_set_error("pi_op_memory_gates: raw gates, biases, a positive cap, the sequences' state and slot words are required"); return -1; }
-    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 20.0 * heads * n_tok, k_memory_gates, dim3((unsigned) heads), dim3(64), 0, (hipStream_t) stream, raw_i, raw_f, stride, bias_i_dev, bias_f_dev, cap, heads, m_state_dev, rec_dev, n_tok,
+    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 20.0 * heads * n_tok, k_memory_gates, dim3((unsigned) heads), dim3((unsigned) std::min(1024, (n_tok + 63) / 64 * 64)), 0, (hipStream_t) stream, raw_i, raw_f, stride, bias_i_dev, bias_f_dev, cap, heads, m_state_dev, rec_dev, n_tok,
                  forget_dev, put_dev, floor_dev, pi_abort_word());
     PI_CHECK_LAUNCH(); return 0;
 }

@@ -10,7 +10,10 @@ shared one) beside the engine's closest model, which is Fasovik at the same widt
 closest model, which is Vikarax at the same width, depth, attention sizes and with a dense feed-forward of the same width.
 
 `bench.py --compare-window [SIZE,...]`: the Rarevik design (one tanh norm per layer, sliding-window attention with pooled far blocks and a sink or with a head gate, clipped routed experts with a
-gated shared one, a repeated run's input matrix) beside the closest model, which is Vikarax at the same width, depth, attention and expert sizes."""
+gated shared one, a repeated run's input matrix) beside the closest model, which is Vikarax at the same width, depth, attention and expert sizes.
+
+`bench.py --compare-streams [SIZE,...]`: the Rerizen design (four residual streams mixed around every sublayer; matrix memories, attention with a query temperature, latent attention in windows behind a
+query latent) beside the closest model, which is Fasovik at the same width, depth, head and latent sizes and with as many feed-forward parameters per token."""
 import ctypes as C
 import json
 import os
@@ -215,6 +218,42 @@ def write_rarevik(folder, size, seed=1):
     return write_random_tensors(folder, cfg, shapes, ones=("norm", "norm1"), seed=seed)
 
 
+def rerizen_ff(size):
+    """a gated dense feed-forward with the parameters a token's chosen experts have in the Fasovik model of the size"""
+    top, ff = SIZES[size][8], SIZES[size][9]
+    return max(64, int(round(2 * top * ff / 3 / 64)) * 64)
+
+
+def write_rerizen(folder, size, seed=1, streams=4):
+    """layers in turn: latent attention in a window, matrix memory, attention with a query temperature, matrix memory (two layers: the first two); window = the Vikarax model's chunk of this size"""
+    width, n_layer, heads, dim, vdim, rank, _, _, _, _, vocab = SIZES[size]
+    kv_heads, window, ff, rot, q_rank = VIKARAX[size][0], VIKARAX[size][2], rerizen_ff(size), dim // 2, width // 2
+    layers, shapes = [], {"embed": (vocab, width), "head": (vocab, width), "final.norm": (width,)}
+    for i in range(n_layer):
+        p, q, hd, hv = "l%d." % i, "l%d.mix." % i, heads * dim, heads * vdim
+        kind = ("latent_attention", "mlstm", "attention", "mlstm")[i % 4]
+        if kind == "mlstm":
+            mx = {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": 15.0}
+            shapes.update({q + "q": (hd, width), q + "k": (hd, width), q + "v": (hv, width), q + "g": (hv, width), q + "o": (width, hv), q + "norm": (hv,), q + "i": (heads, width), q + "i.b": (heads,),
+                           q + "f": (heads, width), q + "f.b": (heads,)})
+        elif kind == "attention":
+            mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "q_temp": {"coef": 0.2, "every": 2048}}
+            for n, rows in (("q", hd), ("k", kv_heads * dim), ("v", kv_heads * vdim)):
+                shapes.update({q + n: (rows, width), q + n + ".b": (rows,)})
+            shapes[q + "o"] = (width, hv)
+        else:
+            mx = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "q_rank": q_rank, "kv_rank": rank, "scale": (dim + rot) ** -0.5, "mask": {"size": window},
+                  "rot": {"dims": rot, "base": 10000.0, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            shapes.update({q + "dq": (q_rank, width), q + "dq.norm": (q_rank,), q + "uq": (heads * (dim + rot), q_rank), q + "dkv": (rank + rot, width), q + "dkv.norm": (rank,), q + "uk": (hd, rank),
+                           q + "uv": (hv, rank), q + "g": (heads, width), q + "o": (width, hv)})
+        layers.append({"type": kind, "mixer": mx, "mlp": {"kind": "dense", "ff": ff}})
+        shapes.update({p + "mlp.gate": (ff, width), p + "mlp.up": (ff, width), p + "mlp.down": (width, ff)})
+        for n in "12":
+            shapes.update({p + "norm" + n: (width,), p + "hc%s.in" % n: (streams,), p + "hc%s.out" % n: (streams,), p + "hc%s.mix" % n: (streams, streams)})
+    cfg = {"architecture": "Rerizen", "vocab": vocab, "width": width, "streams": streams, "norm": {"eps": 1e-5}, "logit_scale": 0.5, "layers": layers}
+    return write_random_tensors(folder, cfg, shapes, ones=("norm", "norm1", "norm2", ".in", ".out"), seed=seed)
+
+
 class KtRow(C.Structure):          # struct pi_kt_row (include/pipeinfer_ops.h)
     _fields_ = [("family", C.c_int32), ("type", C.c_int32), ("n_tok", C.c_int32), ("sampled_dropped", C.c_int32), ("shape_bytes", C.c_uint64), ("launches", C.c_uint64),
                 ("bytes_total", C.c_double), ("sampled", C.c_uint64), ("avg_us", C.c_double), ("avg_sampled_bytes", C.c_double)]
@@ -348,6 +387,27 @@ def main_window(sizes, cache, n_prompt=512, n_decode=64):
     return 0
 
 
+def main_streams(sizes, cache, n_prompt=512, n_decode=64):
+    """Rerizen beside Fasovik at equal sizes; one JSON line per size"""
+    lib = L.load()
+    L.check(lib.pi_device_init(0), "pi_device_init")
+    for size in sizes:
+        width, n_layer, heads, dim, vdim, rank, n_exp, n_id, top, ff, vocab = SIZES[size]
+        rer, fas = os.path.join(cache, "rerizen-" + size), os.path.join(cache, "fasovik-" + size)
+        if not os.path.exists(os.path.join(rer, "model.safetensors")):
+            write_rerizen(rer, size)
+        if not os.path.exists(os.path.join(fas, "model.safetensors")):
+            write_fasovik(fas, size)
+        out = {"size": size, "config": {"width": width, "layers": n_layer, "streams": 4, "heads": heads, "kv_heads": VIKARAX[size][0], "dim": dim, "vdim": vdim, "rot_dim": dim // 2, "q_rank": width // 2, "kv_rank": rank,
+                                       "window": VIKARAX[size][2], "ff": rerizen_ff(size), "vocab": vocab, "n_prompt": n_prompt, "n_decode": n_decode,
+                                       "fasovik": {"experts": n_exp, "identity": n_id, "top": top, "ff": ff}},
+               "rerizen_bf16": measure(lib, rer, n_prompt, n_decode, True),
+               "fasovik_bf16": measure(lib, fas, n_prompt, n_decode, True), "data": "synthetic", "hbm_peak": HBM_PEAK}
+        print(json.dumps(out))
+        sys.stdout.flush()
+    return 0
+
+
 def main(sizes, cache, n_prompt=512, n_decode=64):
     lib = L.load()
     L.check(lib.pi_device_init(0), "pi_device_init")
@@ -376,7 +436,7 @@ def run_phase(design, size, phase, cache, n_prompt=512, n_decode=64):
     L.check(lib.pi_device_init(0), "pi_device_init")
     folder = os.path.join(cache, "%s-%s" % (design, size))
     if not os.path.exists(os.path.join(folder, "model.safetensors")):
-        {"vikarax": write_vikarax, "fasovik": write_fasovik, "rafusun": write_rafusun, "rarevik": write_rarevik}[design](folder, size)
+        {"vikarax": write_vikarax, "fasovik": write_fasovik, "rafusun": write_rafusun, "rarevik": write_rarevik, "rerizen": write_rerizen}[design](folder, size)
     model = LL.Model(folder)
     ctx = LL.Context(model, n_ctx=n_prompt + n_decode + 64, n_batch=n_prompt)
     ctx.set_precision(False)
@@ -397,7 +457,7 @@ def run_phase(design, size, phase, cache, n_prompt=512, n_decode=64):
 if __name__ == "__main__":
     import argparse
     ap = argparse.ArgumentParser(description="one phase of one folder-described design at one size (for `rocprofv3 --kernel-trace --stats -- python3 -m pipeinfer_amd.tools.hybrid_bench ...`)")
-    ap.add_argument("--design", choices=["vikarax", "fasovik", "rafusun", "rarevik"], required=True)
+    ap.add_argument("--design", choices=["vikarax", "fasovik", "rafusun", "rarevik", "rerizen"], required=True)
     ap.add_argument("--size", choices=sorted(SIZES), default="w2048")
     ap.add_argument("--phase", choices=["prefill", "decode"], required=True)
     ap.add_argument("--cache", default=os.environ.get("PIPEINFER_CACHE", "/tmp/pipeinfer_models"))
