@@ -20,9 +20,9 @@ class PipeInferError(RuntimeError):
 
 
 def build(force=False):
-    """compile the HIP extension in-tree (hipcc cross-compiles gfx950 without a GPU)"""
+    """compile the HIP extension in-tree (hipcc cross-compiles gfx950 without a GPU); force: every source again, both libraries"""
     if force or not os.path.exists(SO) or _stale():
-        subprocess.check_call(["make", "-C", os.path.join(PKG, "csrc"), "-j8"], stdout=subprocess.DEVNULL)
+        subprocess.check_call(["make", "-C", os.path.join(PKG, "csrc"), "-j8"] + (["-B", "all", "dense"] if force else []), stdout=subprocess.DEVNULL)
     return SO
 
 
