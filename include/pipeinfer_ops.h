@@ -410,6 +410,28 @@ PI_API int pi_op_latent_attention_rot(const float * q_dev, int64_t q_stride, con
                                       float * scratch_dev, size_t scratch_floats, float * out_dev, int64_t out_stride, const int32_t * dyn_dev, void * stream);
 PI_API size_t pi_op_latent_attention_rot_scratch_floats(int heads, int rank, int rot_dim, int n_tok, int n_kv);
 
+/* ---- operators of plain pre-norm blocks, of latent attention in other pairs with a gate per value, and of differential attention ------------------------------------------------- */
+/* the residual between two sublayers of a pre-norm block: x <- x + y [+ shift] (y, shift [n] nullable) -> x_out (may be x_in), h = x / sqrt(mean(x^2) + eps) * w; rows of x are n floats apart */
+PI_API int pi_op_residual_norm(const float * x_in_dev, const float * y_dev, int64_t y_stride, const float * shift_dev, const float * w_dev, float eps, int n, int n_tok, float * x_out_dev, float * h_out_dev, int64_t h_stride,
+                               void * stream);
+/* pi_op_latent_prepare with the pairs of the rotation as a parameter (pi_rot_pairing) */
+PI_API int pi_op_latent_prepare_ex(const float * p_dev, int64_t p_stride, int q_rank, const float * q_norm_w, int kv_rank, const float * kv_norm_w, int rot_dim, const void * rotary_table, int pairing, float eps,
+                                   const int32_t * pos_dev, int n_tok, float * q_latent_dev, int64_t q_latent_stride, float * cache_dev, const int32_t * dyn_dev, void * stream);
+/* pi_op_latent_attention_rot with the pairs of the rotation and the gate's width as parameters: gate_width 1: one value per head, vdim: one per output value (gate_dev [n_tok][heads * gate_width]) */
+PI_API int pi_op_latent_attention_gated(const float * q_dev, int64_t q_stride, const float * cache_dev, const uint32_t * mask_dev, const pi_weight * w_uk, const pi_weight * w_uv, const float * sink_dev, const float * gate_dev,
+                                        int64_t gate_stride, int gate_act, int gate_width, float scale, int heads, int dim, int rot_dim, int vdim, int rank, const void * rotary_table, int pairing, const int32_t * pos_dev,
+                                        int n_tok, int n_kv, float * scratch_dev, size_t scratch_floats, float * out_dev, int64_t out_stride, const int32_t * dyn_dev, void * stream);
+/* pi_op_qkv_prepare_ex for heads of `maps` query / key maps of `dim` values each over one value of vdim values: q rows [heads][maps][dim], k rows [kv_heads][maps][dim], v rows [kv_heads][vdim]; every map is
+ * turned by itself, nothing is normed.  Cells: k_cache [cells][kv_heads][maps][dim], v_cache [cells][kv_heads][vdim] */
+PI_API int pi_op_qkv_prepare_maps(const float * q_dev, const float * k_dev, const float * v_dev, int64_t stride, int heads, int kv_heads, int maps, int dim, int vdim, const void * rotary_table, int pairing, const int32_t * pos_dev,
+                                  int n_tok, float * q_out_dev, int64_t q_out_stride, float * k_cache_dev, float * v_cache_dev, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream);
+/* Soft-max attention over a window with kept first tokens: a token at position p sees its sequence's cells at positions c <= p with p - c < size (size 0: all) or c < keep_first.
+ * maps = 2 (caches as pi_op_qkv_prepare_maps leaves them): both maps of a head attend by themselves over the same values, a1 and a2; out = R(a1 - lam * a2) * out_mult, R over the head's vdim values with eps.
+ * maps = 1: the plain soft-max times out_mult.  scratch_dev (nullable): pi_op_window_attention_scratch_floats(heads * maps, vdim, n_tok) floats */
+PI_API int pi_op_diff_attention(const float * q_dev, int64_t q_stride, const float * k_cache_dev, const float * v_cache_dev, const int32_t * cell_pos_dev, const uint32_t * mask_dev, const int32_t * pos_dev, float scale, int size,
+                                int keep_first, int maps, float lam, float out_mult, float eps, int heads, int kv_heads, int dim, int vdim, int n_tok, int n_kv, float * scratch_dev, size_t scratch_floats, float * out_dev,
+                                int64_t out_stride, const int32_t * dyn_dev, void * stream);
+
 #ifdef __cplusplus
 }
 #endif

@@ -113,7 +113,7 @@ static bool context_prepare_hybrid(llama_context * ctx, std::string & err) {
     if (hp.n_recurrent() > 0 || hp.pair_buckets > 0) ctx->slots.reset(new state_slots(std::max(1, ctx->n_state_slots)));      // (the previous token of a pair embedding is per-sequence state as well)
     for (size_t i = 0; i < hp.hybrid.size(); i++) {
         const pi_hybrid_layer & H = hp.hybrid[i];
-        if (hp.streams > 0) {                                                  // scratch rows as forward_stream_blocks lays them out
+        if (hp.streams > 0 || hp.pre_norm) {                                   // scratch rows as forward_stream_blocks / forward_pre_norm_blocks lay them out
             if (H.cache_index >= 0) { ctx->lat_off[i] = lat; lat += (size_t) ctx->n_ctx * H.cell_floats(); }
             if (H.kv_from >= 0) ctx->lat_off[i] = ctx->lat_off[(size_t) H.kv_from];
             if (H.state_index >= 0) { ctx->rec_off[i] = rec; rec += (size_t) ctx->slots->size() * H.state_floats(); }
@@ -123,8 +123,8 @@ static bool context_prepare_hybrid(llama_context * ctx, std::string & err) {
                 att_w = std::max(att_w, (size_t) M.heads * (2 * M.vdim + 1) + (size_t) 3 * M.heads + 4);
                 ctx->rec_scratch_floats = std::max(ctx->rec_scratch_floats, pi_op_linear_attention_scratch_floats(M.heads, M.dim, M.vdim + 1, nb, ctx->slots->size()));
             } else if (H.mixer == PI_MIXER_WINDOW_ATTENTION) {
-                att_w = std::max(att_w, (size_t) H.left.heads * (H.left.dim + H.left.vdim));
-                ctx->lat_scratch_floats = std::max(ctx->lat_scratch_floats, pi_op_window_attention_scratch_floats(H.left.heads, H.left.vdim, nb));
+                att_w = std::max(att_w, (size_t) H.left.heads * (H.left.maps * H.left.dim + H.left.vdim) + (H.left.conv > 0 ? (size_t) row_of_4(H.left.channels()) : 0));
+                ctx->lat_scratch_floats = std::max(ctx->lat_scratch_floats, pi_op_window_attention_scratch_floats(H.left.heads * H.left.maps, H.left.vdim, nb));
             } else {
                 att_w = std::max(att_w, (size_t) row_of_4(H.latent.q_rank) + (size_t) H.heads * (H.dim + H.latent.rot_dim) + (size_t) H.heads * H.vdim + 4);
                 ctx->lat_scratch_floats = std::max(ctx->lat_scratch_floats, pi_op_latent_attention_rot_scratch_floats(H.heads, H.kv_rank, H.latent.rot_dim, nb, ctx->n_ctx));
@@ -664,7 +664,7 @@ static bool forward_temp_attention(llama_context * ctx, const pi_hybrid_layer & 
     OP_OK(pi_op_dense(W.w_o, O, hv, n_tok, ctx->h_out, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
     return true;
 }
-static bool forward_latent_window(llama_context * ctx, const pi_hybrid_layer & H, const pi_hybrid_weights & W, size_t il, const float * N, int n_tok, int n_kv) {
+static bool forward_query_latent(llama_context * ctx, const pi_hybrid_layer & H, const pi_hybrid_weights & W, size_t il, const float * N, int n_tok, int n_kv) {
     hipStream_t s = ctx->stream;
     const pi_latent & A = H.latent;
     const int width = ctx->model->hparams.n_embd, ex = ctx->exact, nb = ctx->n_batch, R = A.rot_dim;
@@ -673,10 +673,10 @@ static bool forward_latent_window(llama_context * ctx, const pi_hybrid_layer & H
     float * cache = ctx->lat_cache + ctx->lat_off[il];
     const uint32_t * mask = A.window > 0 ? ctx->window_masks.at(A.window) : ctx->mask_dev;
     OP_OK(pi_op_dense(W.w_in, N, width, n_tok, P, pw, PI_ACT_NONE, pw, PI_ACT_NONE, ex, s));
-    OP_OK(pi_op_latent_prepare(P, pw, A.q_rank, W.q_norm, H.kv_rank, W.mix_norm, R, W.rotary, ctx->model->hparams.f_norm_rms_eps, ctx->pos_dev, n_tok, C, cw, cache, ctx->dyn_dev, s));
+    OP_OK(pi_op_latent_prepare_ex(P, pw, A.q_rank, W.q_norm, H.kv_rank, W.mix_norm, R, W.rotary, A.pairing, ctx->model->hparams.f_norm_rms_eps, ctx->pos_dev, n_tok, C, cw, cache, ctx->dyn_dev, s));
     OP_OK(pi_op_dense(W.w_uq, C, cw, n_tok, Q, qw, PI_ACT_NONE, qw, PI_ACT_NONE, ex, s));
-    OP_OK(pi_op_latent_attention_rot(Q, qw, cache, mask, W.w_uk, W.w_uv, nullptr, A.gated ? P + A.q_rank + H.kv_rank + R : nullptr, pw, PI_ACT_SIGMOID, H.scale, H.heads, H.dim, R, H.vdim, H.kv_rank, W.rotary, ctx->pos_dev, n_tok,
-                                     n_kv, ctx->lat_scratch, ctx->lat_scratch_floats, O, hv, ctx->dyn_dev, s));
+    OP_OK(pi_op_latent_attention_gated(Q, qw, cache, mask, W.w_uk, W.w_uv, W.sink, A.gated ? P + A.q_rank + H.kv_rank + R : nullptr, pw, PI_ACT_SIGMOID, A.gate_width, H.scale, H.heads, H.dim, R, H.vdim, H.kv_rank, W.rotary,
+                                       A.pairing, ctx->pos_dev, n_tok, n_kv, ctx->lat_scratch, ctx->lat_scratch_floats, O, hv, ctx->dyn_dev, s));
     trace(ctx, "lat", (int) il, O, hv, n_tok);
     OP_OK(pi_op_dense(W.w_o, O, hv, n_tok, ctx->h_out, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
     return true;
@@ -706,7 +706,7 @@ static bool forward_stream_blocks(llama_context * ctx, int n_tok, int n_kv) {
         switch (H.mixer) {
             case PI_MIXER_MEMORY:           ok = forward_memory(ctx, H, W, il, N, n_tok); break;
             case PI_MIXER_WINDOW_ATTENTION: ok = forward_temp_attention(ctx, H, W, il, N, n_tok, n_kv); break;
-            case PI_MIXER_LATENT_ATTENTION: ok = forward_latent_window(ctx, H, W, il, N, n_tok, n_kv); break;
+            case PI_MIXER_LATENT_ATTENTION: ok = forward_query_latent(ctx, H, W, il, N, n_tok, n_kv); break;
             default: ctx->last_error = "blocks over residual streams are built for the matrix-memory, attention and latent-attention mixers";
         }
         if (!ok) return false;
@@ -727,6 +727,77 @@ static bool forward_stream_blocks(llama_context * ctx, int n_tok, int n_kv) {
     return true;
 }
 
+// Plain pre-norm blocks (hp.pre_norm), R(u) = u / sqrt(mean(u^2) + eps):   x <- x + mixer(R(x) * w1);  x <- x + ff(R(x) * w2).  A run of layers may repeat with the same tensors (every entry of hp.hybrid is
+// one run, with a cache and state of its own); in front of pass t of the run x <- x + step_t.
+//   differential attention   ONE projection [q | k | v] -> convolution per channel (+ its state) -> rotation of every map, cache store -> soft-max attention of both maps over the window and the kept first
+//                            tokens, their difference normed per head -> W_o
+//   latent attention         forward_query_latent, with a sink and a gate per output value
+//   feed-forward             [gate | up] -> clipped product -> down
+// A sublayer ends in ONE row kernel (pi_op_residual_norm): the sum (with the pass's vector where the next layer opens one) and the norm of what reads it next; behind the last one the model's norm.
+static bool forward_diff_attention(llama_context * ctx, const pi_hybrid_layer & H, const pi_hybrid_weights & W, size_t il, const float * N, int n_tok, int n_kv) {
+    hipStream_t s = ctx->stream;
+    const pi_gate_attention & A = H.left;
+    const int width = ctx->model->hparams.n_embd, ex = ctx->exact, nb = ctx->n_batch, ch = A.channels();
+    const int64_t pw = row_of_4(H.in_rows()), cw = row_of_4(ch), hd = (int64_t) A.heads * A.maps * A.dim, hv = (int64_t) A.heads * A.vdim, gd = (int64_t) A.kv_heads * A.maps * A.dim;
+    float * P = ctx->h_in, * Q = ctx->h_att, * O = Q + (size_t) nb * hd, * C = O + (size_t) nb * hv;
+    float * kc = ctx->lat_cache + ctx->lat_off[il], * vc = kc + (size_t) ctx->n_ctx * gd;
+    OP_OK(pi_op_dense(W.w_in, N, width, n_tok, P, pw, PI_ACT_NONE, pw, PI_ACT_NONE, ex, s));
+    const float * qkv = P; int64_t qs = pw;
+    if (A.conv > 0) { OP_OK(pi_op_causal_conv(P, pw, ch, A.conv, W.conv_w, nullptr, ctx->rec_state + ctx->rec_off[il], ctx->rec_dev, n_tok, PI_ACT_NONE, C, cw, s)); qkv = C; qs = cw; }
+    OP_OK(pi_op_qkv_prepare_maps(qkv, qkv + hd, qkv + hd + gd, qs, A.heads, A.kv_heads, A.maps, A.dim, A.vdim, W.rotary, A.pairing, ctx->pos_dev, n_tok, Q, hd, kc, vc, ctx->cell_pos, ctx->dyn_dev, s));
+    OP_OK(pi_op_diff_attention(Q, hd, kc, vc, ctx->cell_pos, ctx->mask_dev, ctx->pos_dev, A.scale, A.chunk, A.keep_first, A.maps, W.lam, 1.0f - A.diff, ctx->model->hparams.f_norm_rms_eps, A.heads, A.kv_heads, A.dim, A.vdim, n_tok,
+                               n_kv, ctx->lat_scratch, ctx->lat_scratch_floats, O, hv, ctx->dyn_dev, s));
+    trace(ctx, "att", (int) il, O, hv, n_tok);
+    OP_OK(pi_op_dense(W.w_o, O, hv, n_tok, ctx->h_out, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
+    return true;
+}
+static bool forward_pre_norm_blocks(llama_context * ctx, int n_tok, int n_kv) {
+    llama_model * m = ctx->model;
+    const pi_hparams & hp = m->hparams;
+    hipStream_t s = ctx->stream;
+    const int width = hp.n_embd, ex = ctx->exact, nb = ctx->n_batch;
+    const float eps = hp.f_norm_rms_eps;
+    const size_t n_layer = hp.hybrid.size();
+    float * x = ctx->x, * N = ctx->nx, * Y = ctx->h_out, * P = ctx->h_in;
+    // x + y (+ the vector of the pass that run `next` opens) -> x, the norm that run `next` (or the model's output) reads -> N
+    auto step_to = [&](size_t next, const float * y) {
+        const bool last = next == n_layer;
+        const float * w = last ? m->output_norm : m->hweights[(size_t) hp.hybrid[next].weights].norm1, * shift = !last && hp.hybrid[next].loop_entry ? m->loop_step + (size_t) hp.hybrid[next].loop_pass * width : nullptr;
+        if (trace_enabled() && y) {                                            // (the stream as the layer left it)
+            if (pi_op_residual_norm(x, y, width, nullptr, w, eps, width, n_tok, x, N, width, s) != 0) return -1;
+            trace(ctx, "lout", (int) next - 1, x, width, n_tok);
+            y = nullptr;
+        }
+        return pi_op_residual_norm(x, y, width, shift, w, eps, width, n_tok, x, N, width, s);
+    };
+    if (m->pair_embd) OP_OK(pi_op_embed_pair(m->tok_embd, ctx->tokens_dev, n_tok, hp.embed_scale, m->pair_embd, ctx->pair_dev, x, s));
+    else OP_OK(pi_op_embed(m->tok_embd, ctx->tokens_dev, n_tok, hp.embed_scale, x, s));
+    OP_OK(step_to(0, nullptr));
+    for (size_t il = 0; il < n_layer; il++) {
+        const pi_hybrid_layer & H = hp.hybrid[il];
+        const pi_hybrid_weights & W = m->hweights[(size_t) H.weights];
+        bool ok = false;
+        switch (H.mixer) {
+            case PI_MIXER_WINDOW_ATTENTION: ok = forward_diff_attention(ctx, H, W, il, N, n_tok, n_kv); break;
+            case PI_MIXER_LATENT_ATTENTION: ok = forward_query_latent(ctx, H, W, il, N, n_tok, n_kv); break;
+            default: ctx->last_error = "plain pre-norm blocks are built for the window-attention and latent-attention mixers";
+        }
+        if (!ok) return false;
+        if (H.has_mlp) {
+            const int ff = H.ff;
+            float * G = P + (size_t) nb * 2 * ff;
+            OP_OK(pi_op_residual_norm(x, Y, width, nullptr, W.norm2, eps, width, n_tok, x, N, width, s));
+            OP_OK(pi_op_dense(W.ff_up, N, width, n_tok, P, 2 * (int64_t) ff, PI_ACT_NONE, 2 * (int64_t) ff, PI_ACT_NONE, ex, s));
+            OP_OK(pi_op_glu_mul_ex(P, 2 * (int64_t) ff, ff, PI_GLU_CLIPPED, H.glu_limit, -1, n_tok, G, ff, s));
+            OP_OK(pi_op_dense(W.ff_down, G, ff, n_tok, Y, width, PI_ACT_NONE, width, PI_ACT_NONE, ex, s));
+        }
+        OP_OK(step_to(il + 1, Y));
+    }
+    OP_OK(pi_op_dense(m->tok_embd, N, width, n_tok, ctx->logits_dev, hp.n_vocab, PI_ACT_NONE, hp.n_vocab, PI_ACT_NONE, ex, s));
+    OP_OK(pi_op_topk(ctx->logits_dev, hp.n_vocab, n_tok, 8, ctx->topk_ids_dev, ctx->topk_vals_dev, ctx->topk_sum_dev, ctx->topk_scratch_dev, s));
+    return true;
+}
+
 static bool forward_hybrid(llama_context * ctx, int n_tok, int n_kv) {
     llama_model * m = ctx->model;
     const pi_hparams & hp = m->hparams;
@@ -734,6 +805,7 @@ static bool forward_hybrid(llama_context * ctx, int n_tok, int n_kv) {
     if (hp.post_norm) return forward_post_norm_blocks(ctx, n_tok, n_kv);
     if (hp.shared_tanh_norm) return forward_shared_norm_blocks(ctx, n_tok, n_kv);
     if (hp.streams > 0) return forward_stream_blocks(ctx, n_tok, n_kv);
+    if (hp.pre_norm) return forward_pre_norm_blocks(ctx, n_tok, n_kv);
     hipStream_t s = ctx->stream;
     const int width = hp.n_embd, ex = ctx->exact;
     const float eps = hp.f_norm_rms_eps, rm = hp.residual_mult;

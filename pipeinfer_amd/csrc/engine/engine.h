@@ -38,7 +38,9 @@ enum pi_arch { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_BAICHUAN = 2, PI_A
                PI_ARCH_RAREVIK = 12 /* hybrid as well: ONE tanh norm per layer that mixer and feed-forward both read (x <- x + mixer(shift(h)) + ff(h)), a run of layers repeated with the same tensors,
                                        sliding-window attention with pooled far blocks and a learned sink, or with a per-head output gate; clipped gated experts behind a top-logit router */,
                PI_ARCH_RERIZEN = 13 /* hybrid as well: the residual is several streams mixed by small learned matrices around every sublayer; mixers: a normalised matrix memory with exponential gates,
-                                       attention with query temperatures (keys and values of its own or another layer's), latent attention behind a query latent with a rotated part and a window */ };
+                                       attention with query temperatures (keys and values of its own or another layer's), latent attention behind a query latent with a rotated part and a window */,
+               PI_ARCH_LETEVIK = 14 /* hybrid as well: plain pre-norm blocks (x <- x + sublayer(R(x) w)), a hashed pair embedding, a run of layers repeated with the same tensors behind a learned vector per pass;
+                                       mixers: differential attention in a window with kept first tokens behind short convolutions, latent attention with a sink and a gate per output value */ };
 
 // what the reference's build_* functions differ in (llama.cpp:3985-4104 baichuan, 4229-4327 starcoder, 4540-4630 refact, 4632-4725 bloom, 4727-4825 mpt, 4827-4939 stablelm)
 struct pi_block {
@@ -73,13 +75,15 @@ struct pi_gate_attention { int heads = 0, kv_heads = 0, dim = 0, vdim = 0, rot_d
                            int mask_kind = PI_MASK_CHUNK, pool = 0, conv = 0, qk_norm = PI_QK_NORM_FIRST, pairing = PI_PAIR_HALVES; bool v_norm = true;
                            float rot_factor = 1.0f, rot_low = 1.0f, rot_high = 1.0f; int rot_original = 0;
                            bool bias = false; float temp_coef = 0.0f; int temp_every = 0;                       // biases of q, k, v; query temperature (pi_op_qkv_prepare_temp)
-                           int channels() const { return heads * dim + kv_heads * (dim + vdim); }                                  // [q | k | v]
+                           int maps = 1, keep_first = 0; float diff = 0.0f;                                     // query / key maps of `dim` values per head over one value (2: differential heads, diff: the constant in their factor); positions that a window always shows
+                           int cell_width() const { return kv_heads * (maps * dim + vdim); } int channels() const { return heads * maps * dim + cell_width(); }                                  // [q | k | v]
                            int in_rows() const { return channels() + (gated ? heads : 0); }                                       // [q | k | v | gate]
                            int cell_rows() const { return pool > 0 && chunk > 0 && mask_kind == PI_MASK_WINDOW ? 2 : 1; }          // cache rows per cell: the token's own, and the pooled block it completes
                            size_t conv_floats() const { return conv > 1 ? (size_t) (conv - 1) * channels() : 0; } };
 // what a latent attention has besides heads, dim, vdim, kv_rank and scale: a query latent of q_rank values (0: queries straight from the input), rot_dim rotated dimensions per query head and ONE rotated key
-// part of that size per cell, its angle steps stretched along a ramp (rot_original > 0: pi_rotary_table_create_ramp), a window of positions (0: all), a per-head sigmoid gate, a learned sink
-struct pi_latent { int q_rank = 0, rot_dim = 0, window = 0; bool gated = false, sink = true; float rot_base = 10000.0f, rot_factor = 1.0f, rot_fast = 1.0f, rot_slow = 1.0f; int rot_original = 0; };
+// part of that size per cell, its angle steps stretched along a ramp (rot_original > 0: pi_rotary_table_create_ramp), a window of positions (0: all), a sigmoid gate of gate_width values per head (1, or vdim: one per
+// output value), a learned sink
+struct pi_latent { int q_rank = 0, rot_dim = 0, window = 0; bool gated = false, sink = true; float rot_base = 10000.0f, rot_factor = 1.0f, rot_fast = 1.0f, rot_slow = 1.0f; int rot_original = 0, pairing = PI_PAIR_NEIGHBOURS, gate_width = 1; };
 // normalised matrix memory: q, k (heads x dim), v and an output gate (heads x vdim), an input and a forget gate per head, both capped; per sequence and head a [dim][vdim] matrix with the decayed sum of the
 // keys as one more column, and the running maximum of the log gates
 struct pi_memory { int heads = 0, dim = 0, vdim = 0; float cap = 1.0f;
@@ -102,7 +106,7 @@ enum pi_mlp_kind { PI_MLP_NONE = 0, PI_MLP_MOE_RELU_SQR = 1 /* routed by a soft-
                    PI_MLP_MOE_GLU = 3 /* routed by sigmoid scores inside the best groups, experts silu(gate) * up, an optional shared expert */, PI_MLP_DENSE_GEGLU = 4 /* down (gelu_tanh(gate) * up) */,
                    PI_MLP_DENSE_GELU = 5 /* down gelu(up), the erf form */, PI_MLP_MOE_CLIPPED = 6 /* the `top` largest router logits (+ bias), soft-max over those; experts down(g sigmoid(1.702 g) (u + 1)) with
                                                                                                        g = min(gate, limit), u = clip(up, +-limit); an optional shared expert of the same form times a per-token sigmoid gate */,
-                   PI_MLP_DENSE_SWIGLU = 7 /* down (silu(gate) * up) */ };
+                   PI_MLP_DENSE_SWIGLU = 7 /* down (silu(gate) * up) */, PI_MLP_DENSE_CLIPPED = 8 /* the clipped expert's form, dense */ };
 struct pi_hybrid_layer {
     pi_mixer_kind mixer = PI_MIXER_LATENT_ATTENTION;
     int weights = 0;                                  // index of the layer that owns the tensors (its own index unless shared)
@@ -114,13 +118,14 @@ struct pi_hybrid_layer {
     pi_latent latent; pi_memory memory; int kv_from = -1;                                   // PI_MIXER_LATENT_ATTENTION; PI_MIXER_MEMORY; PI_MIXER_WINDOW_ATTENTION: the layer whose keys and values it reads (-1: its own)
     bool has_mlp = false; int n_expert = 0, n_identity = 0, top = 0, ff = 0;
     pi_mlp_kind mlp = PI_MLP_NONE; int route_groups = 0, route_keep = 0, shared_ff = 0;     // (has_mlp <=> mlp != PI_MLP_NONE)
-    float glu_limit = 0.0f, shared_limit = 0.0f;      // clipped experts: the bound on gate (from above) and up (both sides); 0: none
+    float glu_limit = 0.0f, shared_limit = 0.0f;      // clipped hidden layers (dense, experts): the bound on gate (from above) and up (both sides); 0: none
     int name_index = -1;                              // the layer of the description whose names the tensors carry (a repeated run lists a layer several times; -1: the entry's own index)
-    bool loop_entry = false;                          // first layer of a repeated run: x <- W_in [x ; embedding row] in front of it
+    bool loop_entry = false;                          // first layer of a repeated run: x <- W_in [x ; embedding row] in front of it (shared_tanh_norm), or x <- x + the learned vector of the pass (pre_norm)
+    int loop_pass = 0;                                // the number of that pass
     int cache_index = -1, state_index = -1;           // ordinal among the layers that keep a per-cell cache / a recurrent state
-    int in_rows() const { return mixer == PI_MIXER_MEMORY ? memory.in_rows() : mixer == PI_MIXER_LATENT_ATTENTION && latent.q_rank > 0 ? latent.q_rank + kv_rank + latent.rot_dim + (latent.gated ? heads : 0) : kv_from >= 0 ? left.heads * left.dim : mixer == PI_MIXER_CHANNEL_DELTA ? delta.in_rows() : mixer == PI_MIXER_PARALLEL_SHIFT || mixer == PI_MIXER_WINDOW_ATTENTION ? left.in_rows() : mixer == PI_MIXER_PARALLEL ? left.in_rows() + right.in_rows() : mixer == PI_MIXER_LIGHTNING ? 2 * heads * dim + 2 * heads * vdim : heads * dim + kv_rank; }     // rows of the fused input projection
+    int in_rows() const { return mixer == PI_MIXER_MEMORY ? memory.in_rows() : mixer == PI_MIXER_LATENT_ATTENTION && latent.q_rank > 0 ? latent.q_rank + kv_rank + latent.rot_dim + (latent.gated ? heads * latent.gate_width : 0) : kv_from >= 0 ? left.heads * left.dim : mixer == PI_MIXER_CHANNEL_DELTA ? delta.in_rows() : mixer == PI_MIXER_PARALLEL_SHIFT || mixer == PI_MIXER_WINDOW_ATTENTION ? left.in_rows() : mixer == PI_MIXER_PARALLEL ? left.in_rows() + right.in_rows() : mixer == PI_MIXER_LIGHTNING ? 2 * heads * dim + 2 * heads * vdim : heads * dim + kv_rank; }     // rows of the fused input projection
     int out_cols() const { return mixer == PI_MIXER_CHANNEL_DELTA ? delta.heads * delta.vdim : mixer == PI_MIXER_WINDOW_ATTENTION ? left.heads * left.vdim : mixer == PI_MIXER_PARALLEL_SHIFT ? std::max(left.heads * left.vdim, shift.inner()) : mixer == PI_MIXER_PARALLEL ? std::max(left.heads * left.vdim, right.inner()) : heads * vdim; }                                                   // widest input of an output projection
-    size_t cell_floats() const { return mixer == PI_MIXER_CHANNEL_DELTA || kv_from >= 0 ? 0 : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) left.cell_rows() * left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_PARALLEL || mixer == PI_MIXER_PARALLEL_SHIFT ? (size_t) left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_LATENT_ATTENTION ? (size_t) kv_rank + latent.rot_dim : 0; }   // cached per cell
+    size_t cell_floats() const { return mixer == PI_MIXER_CHANNEL_DELTA || kv_from >= 0 ? 0 : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) left.cell_rows() * left.cell_width() : mixer == PI_MIXER_PARALLEL || mixer == PI_MIXER_PARALLEL_SHIFT ? (size_t) left.kv_heads * (left.dim + left.vdim) : mixer == PI_MIXER_LATENT_ATTENTION ? (size_t) kv_rank + latent.rot_dim : 0; }   // cached per cell
     size_t state_floats() const { return mixer == PI_MIXER_MEMORY ? memory.state_floats() : mixer == PI_MIXER_WINDOW_ATTENTION ? (size_t) shift.width + left.conv_floats() : mixer == PI_MIXER_CHANNEL_DELTA ? delta.state_floats() : mixer == PI_MIXER_PARALLEL_SHIFT ? shift.state_floats() : mixer == PI_MIXER_PARALLEL ? right.state_floats() : mixer == PI_MIXER_LIGHTNING ? (size_t) heads * dim * vdim : 0; }                       // kept per sequence
     // a layer's per-sequence state has up to two parts, each stored [slots][part]: the recurrence's matrices, then the convolution's last inputs / the previous token's input / the gates' running maximum
     void state_parts(size_t parts[2]) const {
@@ -146,6 +151,7 @@ struct pi_hybrid_weights {                            // the tensors of a layer 
     // residual streams: per sublayer the factors of its input [streams], of its result [streams] and the mixing matrix [from][to]; memory: w_in = rows [q | k | v | g | i | f], the gates' biases [i | f]
     // (gate_bias); attention: the biases of its input rows (in_bias); latent attention: w_in = rows [dq | dkv | g], w_uq, the query latent's norm (q_norm)
     float * hc_in[2] = { nullptr, nullptr }, * hc_out[2] = { nullptr, nullptr }, * hc_mix[2] = { nullptr, nullptr }, * gate_bias = nullptr, * in_bias = nullptr; pi_weight * w_uq = nullptr;
+    float lam = 0.0f;                                 // differential heads: the factor of the second map, e^(lq1 . lk1) - e^(lq2 . lk2) + diff (one number for the layer, kept on the host)
     pi_weight * w_a2 = nullptr, * w_g2 = nullptr, * w_r = nullptr, * w_k = nullptr, * w_v = nullptr, * w_g = nullptr, * w_w1 = nullptr, * w_w2 = nullptr, * w_o2 = nullptr;
     bool loaded = false;
 };
@@ -168,7 +174,9 @@ struct pi_hparams {
     bool shared_tanh_norm = false;
     // ... or `streams` copies of the residual, mixed around every sublayer: u = in . X -> R(u) * w -> sublayer -> X <- mix^T X + out y; the logits times logit_scale
     int streams = 0; float logit_scale = 1.0f;
-    bool hybrid_arch() const { return arch == PI_ARCH_FASOVIK || arch == PI_ARCH_VIKARAX || arch == PI_ARCH_RAFUSUN || arch == PI_ARCH_RAREVIK || arch == PI_ARCH_RERIZEN; }
+    // ... or the plain pre-norm block: x <- x + sublayer(R(x) w); loop_passes > 0: a repeated run of layers with a learned vector per pass
+    bool pre_norm = false; int loop_passes = 0;
+    bool hybrid_arch() const { return arch == PI_ARCH_FASOVIK || arch == PI_ARCH_VIKARAX || arch == PI_ARCH_RAFUSUN || arch == PI_ARCH_RAREVIK || arch == PI_ARCH_RERIZEN || arch == PI_ARCH_LETEVIK; }
     int n_latent() const { int n = 0; for (const auto & l : hybrid) n += l.cache_index >= 0; return n; }
     int n_recurrent() const { int n = 0; for (const auto & l : hybrid) n += l.state_index >= 0; return n; }
     int head_dim() const { return n_embd / n_head; }
@@ -197,6 +205,7 @@ struct llama_model {
     uint64_t n_elements = 0, n_bytes = 0;
     pi_weight * pair_embd = nullptr;                                                               // hashed pair embedding [pair_buckets + 1][n_embd]
     pi_weight * tok_embd = nullptr, * output = nullptr, * pos_embd = nullptr;                 // pos_embd: StarCoder's learned positions (llama.cpp:4251-4255)
+    float * loop_step = nullptr;                                                                 // repeated runs of pre-norm blocks: [passes][n_embd]
     float * output_norm_alpha = nullptr;                                                         // tanh norms: the final norm's scalar (one float on the device)
     float * output_norm = nullptr, * output_norm_b = nullptr, * tok_norm = nullptr, * tok_norm_b = nullptr;   // tok_norm: Bloom's LayerNorm on the embeddings (llama.cpp:4650-4654)
     float * alibi_slopes = nullptr;                                                              // f32 [n_head] on the device when block.alibi > 0

@@ -196,8 +196,9 @@ size_t llama_model::stage_weight_bytes(int l0, int l1, bool first, bool last, in
                 b += 4 * 4 * w + (H.has_mlp ? 6 * (size_t) H.ff * w : 0);
                 continue;
             }
-            if (hparams.streams > 0) {                                         // the projections and their biases, the up-projections of the latents, the norms' vectors, the dense feed-forward
+            if (hparams.streams > 0 || hparams.pre_norm) {                     // the projections and their biases, convolution taps, the up-projections of the latents, the norms' vectors, the dense feed-forward
                 b += 2 * ((size_t) H.in_rows() + H.out_cols()) * w + 4 * (size_t) (H.has_mlp ? 2 : 1) * w + (H.has_mlp ? 6 * (size_t) H.ff * w : 0);
+                if (H.mixer == PI_MIXER_WINDOW_ATTENTION) b += 4 * (size_t) H.left.channels() * H.left.conv;
                 if (H.mixer == PI_MIXER_LATENT_ATTENTION) b += 2 * (size_t) H.heads * ((size_t) H.latent.q_rank * (H.dim + H.latent.rot_dim) + (size_t) H.kv_rank * (H.dim + H.vdim));
                 continue;
             }
@@ -325,7 +326,7 @@ extern "C" enum llama_vocab_type llama_vocab_type(const struct llama_model * m) 
 extern "C" uint64_t llama_model_size(const struct llama_model * m) { return m->n_bytes; }
 extern "C" uint64_t llama_model_n_params(const struct llama_model * m) { return m->n_elements; }
 extern "C" int llama_model_desc(const struct llama_model * m, char * buf, size_t n) {
-    static const char * names[] = { "llama", "falcon", "baichuan", "starcoder", "refact", "bloom", "mpt", "stablelm", "persimmon", "fasovik", "vikarax", "rafusun", "rarevik", "rerizen" };
+    static const char * names[] = { "llama", "falcon", "baichuan", "starcoder", "refact", "bloom", "mpt", "stablelm", "persimmon", "fasovik", "vikarax", "rafusun", "rarevik", "rerizen", "letevik" };
     return snprintf(buf, n, "%s %s", names[m->hparams.arch], m->name.c_str());
 }
 

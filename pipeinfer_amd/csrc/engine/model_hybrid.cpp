@@ -25,6 +25,11 @@
 // q_temp.coef / q_temp.every, kv_from (optional: the layer whose keys and values it reads) } } or { type: "latent_attention", mixer: { heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot.dims / rot.base /
 // rot.scaling.{factor, original, fast, slow}, mask.size } }, mlp: null | { kind: "dense", ff }.  Tensors: embed, head, final.norm, l<i>.norm1 / norm2, l<i>.hc1 / hc2.{in, out, mix}, l<i>.mix.{q, k, v, g, o, norm, i, i.b,
 // f, f.b} or l<i>.mix.{q, k, v (+ .b), o} or l<i>.mix.{dq, dq.norm, uq, dkv, dkv.norm, uk, uv, g, o}, l<i>.mlp.{gate, up, down}.
+//
+// Letevik (same files, other keys): vocab, width, norm.eps, embedding.bigram.{buckets, mul_prev, mul_cur}, loop.{start, stop, times} (optional, as Rarevik's), layers[]: { type: "attention", mixer: { heads, kv_heads,
+// dim, vdim, scale, conv, diff, rot.dims / rot.base, mask.size / mask.keep_first } } or { type: "latent_attention", mixer: { heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, rot.dims / rot.base } }, mlp: null |
+// { kind: "dense", ff, limit }.  Tensors: embed (also the output matrix), bigram, loop.step, final.norm, l<i>.norm1 / norm2, l<i>.mix.{q, k, v (+ .conv), lq1, lk1, lq2, lk2, o} or l<i>.mix.{dq, dq.norm, uq, dkv,
+// dkv.norm, uk, uv, sink, g, o}, l<i>.mlp.{gate, up, down}.
 #include "engine.h"
 #include "json.h"
 
@@ -116,6 +121,13 @@ struct loader {
         }
         return vector_f32(v);
     }
+    bool host_vector(const std::string & name, int64_t n, std::vector<double> & out) {       // a vector that only the host needs
+        const pi::st_tensor * t = get(name, { n });
+        if (!t) return false;
+        out.resize((size_t) n);
+        for (int64_t i = 0; i < n; i++) out[(size_t) i] = bf16_to_f32(((const uint16_t *) t->data)[i]);
+        return true;
+    }
     float * scalar(const std::string & name) {                                  // a tensor without dimensions: one float on the device
         const pi::st_tensor * t = get(name, {});
         if (!t) return nullptr;
@@ -195,6 +207,40 @@ static bool read_vikarax_config(const pi::json & cfg, pi_hparams & hp, std::stri
     return true;
 }
 
+// a pair embedding's table and multipliers, where the description has one
+static bool read_pair_embedding(const pi::json & cfg, pi_hparams & hp, std::string & what) {
+    if (!cfg.at("embedding.bigram") || cfg.at("embedding.bigram")->is_null()) return true;
+    if (int_at(cfg, "embedding.bigram.buckets", hp.pair_buckets) && int_at(cfg, "embedding.bigram.mul_prev", hp.pair_mul_prev) && int_at(cfg, "embedding.bigram.mul_cur", hp.pair_mul_cur) && hp.pair_buckets > 0) return true;
+    what = "embedding.bigram needs a positive 'buckets', 'mul_prev' and 'mul_cur'"; return false;
+}
+
+// the order the layers run in: [0, start) once, [start, stop) `times` times, [stop, n) once.  Every entry of the run list is a layer of its own to the context (cache, state); its tensors are those of
+// the first run of the same description.  A layer without a state (has_state false) takes no slot rows
+static bool expand_runs(const pi::json & cfg, const std::vector<pi_hybrid_layer> & desc, pi_hparams & hp, int & passes, std::string & what) {
+    const int n_desc = (int) desc.size();
+    int start = n_desc, stop = n_desc, times = 1;
+    passes = 0;
+    if (cfg.at("loop") && !cfg.at("loop")->is_null()) {
+        if (!int_at(cfg, "loop.start", start) || !int_at(cfg, "loop.stop", stop) || !int_at(cfg, "loop.times", times) || start > stop || stop > n_desc || times > 4096) { what = "'loop' needs 0 <= start <= stop <= layers and 'times'"; return false; }
+        passes = times;
+    }
+    std::vector<int> first_run((size_t) n_desc, -1);
+    auto add = [&](int i, int pass) {
+        pi_hybrid_layer H = desc[(size_t) i];
+        const int r = (int) hp.hybrid.size();
+        if (first_run[(size_t) i] < 0) first_run[(size_t) i] = r;
+        H.weights = first_run[(size_t) i]; H.loop_entry = pass >= 0; H.loop_pass = std::max(pass, 0); H.cache_index = r; H.state_index = H.state_floats() > 0 ? r : -1;
+        hp.hybrid.push_back(std::move(H));
+    };
+    for (int i = 0; i < start; i++) add(i, -1);
+    for (int k = 0; k < times; k++) for (int i = start; i < stop; i++) add(i, i == start ? k : -1);
+    for (int i = stop; i < n_desc; i++) add(i, -1);
+    if (hp.hybrid.empty()) { what = "no layer runs"; return false; }
+    hp.n_layer = (int) hp.hybrid.size();
+    hp.n_head = hp.n_head_kv = 1; hp.n_ctx_train = 0;
+    return true;
+}
+
 // Rafusun: layers of two kinds (a delta-rule mixer, or attention beside time mixing), an optional gated dense feed-forward, the norm after the sum
 static bool read_rafusun_config(const pi::json & cfg, const pi::safetensors_file * st, pi_hparams & hp, std::string & what) {
     using pi::json;
@@ -204,9 +250,7 @@ static bool read_rafusun_config(const pi::json & cfg, const pi::safetensors_file
     if (!num_at(cfg, "postln_alpha", d)) { what = "no 'postln_alpha'"; return false; }
     hp.post_alpha = (float) d; hp.post_norm = hp.own_head = true;
     hp.embed_scale = num_at(cfg, "embedding.scale", d) ? (float) d : 1.0f;
-    if (cfg.at("embedding.bigram") && !cfg.at("embedding.bigram")->is_null()) {
-        if (!int_at(cfg, "embedding.bigram.buckets", hp.pair_buckets) || !int_at(cfg, "embedding.bigram.mul_prev", hp.pair_mul_prev) || !int_at(cfg, "embedding.bigram.mul_cur", hp.pair_mul_cur) || hp.pair_buckets < 1) { what = "embedding.bigram needs a positive 'buckets', 'mul_prev' and 'mul_cur'"; return false; }
-    }
+    if (!read_pair_embedding(cfg, hp, what)) return false;
     const json * layers = cfg.find("layers");
     if (!layers || !layers->is_arr() || layers->arr.empty()) { what = "'layers' must be a non-empty list"; return false; }
     hp.n_layer = (int) layers->arr.size();
@@ -326,26 +370,32 @@ static bool read_rarevik_config(const pi::json & cfg, pi_hparams & hp, std::stri
         }
         desc.push_back(std::move(H));
     }
-    // the order the layers run in: [0, start) once, [start, stop) `times` times, [stop, n) once.  Every entry of the run list is a layer of its own to the context (cache, state); its tensors are those of
-    // the first run of the same description
-    int start = n_desc, stop = n_desc, times = 1;
-    if (cfg.at("loop") && !cfg.at("loop")->is_null()) {
-        if (!int_at(cfg, "loop.start", start) || !int_at(cfg, "loop.stop", stop) || !int_at(cfg, "loop.times", times) || start > stop || stop > n_desc || times > 4096) { what = "'loop' needs 0 <= start <= stop <= layers and 'times'"; return false; }
+    int passes = 0;
+    return expand_runs(cfg, desc, hp, passes, what);
+}
+
+// latent attention behind a query latent: ranks, scale, the rotated part with its (possibly stretched) angle steps; heads, dim and vdim are read already
+static bool read_query_latent_attention(const pi::json & jl, pi_hybrid_layer & H, std::string & what) {
+    double d;
+    auto given = [&](const char * path) { const pi::json * v = jl.at(path); return v && !v->is_null(); };
+    auto bad = [&](const char * w) { what = w; return false; };
+    H.mixer = PI_MIXER_LATENT_ATTENTION;
+    pi_latent & A = H.latent;
+    A.gated = true;
+    if (!int_at(jl, "mixer.q_rank", A.q_rank) || !int_at(jl, "mixer.kv_rank", H.kv_rank) || A.q_rank < 1 || H.kv_rank < 1 || H.kv_rank > 1024 || !num_at(jl, "mixer.scale", d)) return bad("latent_attention needs positive 'q_rank', 'kv_rank' (at most 1024) and 'scale'");
+    H.scale = (float) d;
+    if (given("mixer.rot_dim") && !int_at(jl, "mixer.rot_dim", A.rot_dim)) return bad("mixer.rot_dim must be an integer");
+    int dims = 0;
+    if (A.rot_dim > 0) {
+        if ((A.rot_dim & 1) || !int_at(jl, "mixer.rot.dims", dims) || dims != A.rot_dim || !num_at(jl, "mixer.rot.base", d) || d <= 0) return bad("latent_attention rotates its whole 'rot_dim' part: an even 'rot_dim', 'rot.dims' equal to it and a positive 'rot.base'");
+        A.rot_base = (float) d;
+        if (given("mixer.rot.scaling")) {
+            double f, fast, slow;
+            if (!num_at(jl, "mixer.rot.scaling.factor", f) || !int_at(jl, "mixer.rot.scaling.original", A.rot_original) || !num_at(jl, "mixer.rot.scaling.fast", fast) || !num_at(jl, "mixer.rot.scaling.slow", slow) ||
+                f <= 0 || fast <= 0 || slow <= 0 || A.rot_original < 1 || d == 1) return bad("mixer.rot.scaling needs positive 'factor', 'original', 'fast' and 'slow' and a 'rot.base' other than 1");
+            A.rot_factor = (float) f; A.rot_fast = (float) fast; A.rot_slow = (float) slow;
+        }
     }
-    std::vector<int> first_run((size_t) n_desc, -1);
-    auto add = [&](int i, bool entry) {
-        pi_hybrid_layer H = desc[(size_t) i];
-        const int r = (int) hp.hybrid.size();
-        if (first_run[(size_t) i] < 0) first_run[(size_t) i] = r;
-        H.weights = first_run[(size_t) i]; H.loop_entry = entry; H.cache_index = r; H.state_index = r;
-        hp.hybrid.push_back(std::move(H));
-    };
-    for (int i = 0; i < start; i++) add(i, false);
-    for (int k = 0; k < times; k++) for (int i = start; i < stop; i++) add(i, i == start);
-    for (int i = stop; i < n_desc; i++) add(i, false);
-    if (hp.hybrid.empty()) { what = "no layer runs"; return false; }
-    hp.n_layer = (int) hp.hybrid.size();
-    hp.n_head = hp.n_head_kv = 1; hp.n_ctx_train = 0;
     return true;
 }
 
@@ -401,24 +451,10 @@ static bool read_rerizen_config(const pi::json & cfg, pi_hparams & hp, std::stri
                 if (J.mixer != PI_MIXER_WINDOW_ATTENTION || J.kv_from >= 0 || J.left.kv_heads != A.kv_heads || J.left.dim != A.dim || J.left.vdim != A.vdim) return bad("'kv_from' must name an attention layer with keys and values of its own, of this layer's sizes");
             } else H.cache_index = n_cache++;
         } else if (type->str == "latent_attention") {
-            H.mixer = PI_MIXER_LATENT_ATTENTION;
-            pi_latent & A = H.latent;
-            A.sink = false; A.gated = true;
-            if (!int_at(jl, "mixer.q_rank", A.q_rank) || !int_at(jl, "mixer.kv_rank", H.kv_rank) || A.q_rank < 1 || H.kv_rank < 1 || H.kv_rank > 1024 || !num_at(jl, "mixer.scale", d)) return bad("latent_attention needs positive 'q_rank', 'kv_rank' (at most 1024) and 'scale'");
-            H.scale = (float) d;
-            if (given("mixer.rot_dim") && !int_at(jl, "mixer.rot_dim", A.rot_dim)) return bad("mixer.rot_dim must be an integer");
-            int dims = 0;
-            if (A.rot_dim > 0) {
-                if ((A.rot_dim & 1) || !int_at(jl, "mixer.rot.dims", dims) || dims != A.rot_dim || !num_at(jl, "mixer.rot.base", d) || d <= 0 || d == 1) return bad("latent_attention rotates its whole 'rot_dim' part: an even 'rot_dim', 'rot.dims' equal to it and a positive 'rot.base' other than 1");
-                A.rot_base = (float) d;
-                if (given("mixer.rot.scaling")) {
-                    double f, fast, slow;
-                    if (!num_at(jl, "mixer.rot.scaling.factor", f) || !int_at(jl, "mixer.rot.scaling.original", A.rot_original) || !num_at(jl, "mixer.rot.scaling.fast", fast) || !num_at(jl, "mixer.rot.scaling.slow", slow) ||
-                        f <= 0 || fast <= 0 || slow <= 0 || A.rot_original < 1) return bad("mixer.rot.scaling needs positive 'factor', 'original', 'fast' and 'slow'");
-                    A.rot_factor = (float) f; A.rot_fast = (float) fast; A.rot_slow = (float) slow;
-                }
-            }
-            if (given("mixer.mask") && (!int_at(jl, "mixer.mask.size", A.window) || A.window < 1)) return bad("mixer.mask needs a positive 'size'");
+            std::string w;
+            if (!read_query_latent_attention(jl, H, w)) return bad(w);
+            H.latent.sink = false;
+            if (given("mixer.mask") && (!int_at(jl, "mixer.mask.size", H.latent.window) || H.latent.window < 1)) return bad("mixer.mask needs a positive 'size'");
             H.cache_index = n_cache++;
         } else return bad("mixer type '" + type->str + "' is unknown (mlstm, attention, latent_attention)");
         if (jl.has("mlp")) {
@@ -430,6 +466,62 @@ static bool read_rerizen_config(const pi::json & cfg, pi_hparams & hp, std::stri
         hp.hybrid.push_back(std::move(H));
     }
     return true;
+}
+
+// Letevik: pre-norm blocks; differential attention in windows with kept first tokens behind short convolutions, latent attention with a sink and a gate per value; a run of layers may repeat
+static bool read_letevik_config(const pi::json & cfg, pi_hparams & hp, std::string & what) {
+    using pi::json;
+    double d;
+    if (!num_at(cfg, "norm.eps", d)) { what = "no 'norm.eps'"; return false; }
+    hp.f_norm_eps = hp.f_norm_rms_eps = (float) d;
+    if (hp.n_embd > 16384) { what = "'width' above 16384"; return false; }
+    hp.pre_norm = true;
+    if (!read_pair_embedding(cfg, hp, what)) return false;
+    const json * layers = cfg.find("layers");
+    if (!layers || !layers->is_arr() || layers->arr.empty()) { what = "'layers' must be a non-empty list"; return false; }
+    std::vector<pi_hybrid_layer> desc;
+    for (int i = 0; i < (int) layers->arr.size(); i++) {
+        const json & jl = layers->arr[(size_t) i];
+        auto bad = [&](const std::string & w) { what = "layers[" + std::to_string(i) + "]: " + w; return false; };
+        auto given = [&](const char * path) { const json * v = jl.at(path); return v && !v->is_null(); };
+        pi_hybrid_layer H;
+        H.name_index = i;
+        const json * type = jl.find("type");
+        if (!type || !type->is_str()) return bad("no 'type'");
+        if (!int_at(jl, "mixer.heads", H.heads) || !int_at(jl, "mixer.dim", H.dim) || !int_at(jl, "mixer.vdim", H.vdim) || H.heads < 1 || H.dim < 1 || H.vdim < 1) return bad("mixer needs positive 'heads', 'dim', 'vdim'");
+        if (type->str == "attention") {
+            H.mixer = PI_MIXER_WINDOW_ATTENTION;
+            pi_gate_attention & A = H.left;
+            A.heads = H.heads; A.dim = H.dim; A.vdim = H.vdim; A.maps = 2;
+            if (!int_at(jl, "mixer.kv_heads", A.kv_heads) || A.kv_heads < 1 || A.heads % A.kv_heads) return bad("attention needs 'kv_heads', a divisor of heads");
+            if (!num_at(jl, "mixer.scale", d)) return bad("attention needs 'scale'");
+            A.scale = (float) d; A.weights = PI_WEIGHTS_SOFTMAX; A.gated = false; A.v_norm = false; A.qk_norm = PI_QK_NORM_NONE; A.pairing = PI_PAIR_NEIGHBOURS; A.mask_kind = PI_MASK_WINDOW;
+            if (!num_at(jl, "mixer.diff", d)) return bad("attention needs 'diff'");
+            A.diff = (float) d;
+            if (given("mixer.conv") && (!int_at(jl, "mixer.conv", A.conv) || A.conv < 1 || A.conv > 64)) return bad("mixer.conv must lie between 1 and 64");
+            if (given("mixer.rot")) {
+                if (!int_at(jl, "mixer.rot.dims", A.rot_dims) || !num_at(jl, "mixer.rot.base", d) || (A.rot_dims & 1) || A.rot_dims > A.dim || d <= 0) return bad("mixer.rot needs an even 'dims' <= dim and a positive 'base'");
+                A.rot_base = (float) d;
+            }
+            if (given("mixer.mask")) {
+                if (!int_at(jl, "mixer.mask.size", A.chunk) || A.chunk < 1) return bad("mixer.mask needs a positive 'size'");
+                if (given("mixer.mask.keep_first") && !int_at(jl, "mixer.mask.keep_first", A.keep_first)) return bad("mixer.mask.keep_first must not be negative");
+            }
+        } else if (type->str == "latent_attention") {
+            std::string w;
+            if (!read_query_latent_attention(jl, H, w)) return bad(w);
+            H.latent.sink = true; H.latent.gate_width = H.vdim; H.latent.pairing = PI_PAIR_HALVES;
+        } else return bad("mixer type '" + type->str + "' is unknown (attention, latent_attention)");
+        if (jl.has("mlp")) {
+            const json * kind = jl.at("mlp.kind");
+            if (!kind || !kind->is_str() || kind->str != "dense") return bad("feed-forward kind must be 'dense'");
+            if (!int_at(jl, "mlp.ff", H.ff) || H.ff < 1) return bad("a dense mlp needs 'ff'");
+            if (given("mlp.limit")) { if (!num_at(jl, "mlp.limit", d) || d <= 0) return bad("mlp.limit must be positive"); H.glu_limit = (float) d; }
+            H.mlp = PI_MLP_DENSE_CLIPPED; H.has_mlp = true;
+        }
+        desc.push_back(std::move(H));
+    }
+    return expand_runs(cfg, desc, hp, hp.loop_passes, what);
 }
 
 // the rotation table of a layer, over n_pos positions
@@ -453,10 +545,11 @@ bool llama_model::ensure_loaded_hybrid(int n_positions, std::string & err) {
     }
     if (hp.own_head && !output) {
         if (!(output = L.matrix({ { "head", hp.n_vocab } }, width))) return false;
-        if (!hp.post_norm && hp.streams == 0 && !(output_norm_b = L.vector("final.norm.b", width))) return false;
+        if (hp.pre_post_norm && !(output_norm_b = L.vector("final.norm.b", width))) return false;
     }
     if (hp.shared_tanh_norm && !output_norm_alpha && (!(output_norm_b = L.vector("final.norm.b", width)) || !(output_norm_alpha = L.scalar("final.norm.alpha")))) return false;
     if (hp.pair_buckets > 0 && !pair_embd && !(pair_embd = L.matrix({ { "bigram", (int64_t) hp.pair_buckets + 1 } }, width))) return false;
+    if (hp.pre_norm && hp.loop_passes > 0 && !loop_step && !(loop_step = L.vector2("loop.step", hp.loop_passes, width))) return false;
     for (size_t i = 0; i < hp.hybrid.size(); i++) {
         const pi_hybrid_layer & H = hp.hybrid[i];
         pi_hybrid_weights & W = hweights[i];
@@ -467,13 +560,13 @@ bool llama_model::ensure_loaded_hybrid(int n_positions, std::string & err) {
         }
         if (H.weights != (int) i || W.loaded) continue;
         const std::string p = "l" + std::to_string(H.name_index >= 0 ? H.name_index : (int) i) + ".";
-        if (hp.streams > 0) {                                              // per sublayer a norm and the streams' factors
+        if (hp.streams > 0 || hp.pre_norm) {                               // per sublayer a norm (and the streams' factors)
             const std::string m = p + "mix.";
             const int n_sub = H.has_mlp ? 2 : 1;
             for (int q = 0; q < n_sub; q++) {
                 const std::string c = p + (q ? "hc2." : "hc1.");
-                if (!((q ? W.norm2 : W.norm1) = L.vector(p + (q ? "norm2" : "norm1"), width)) || !(W.hc_in[q] = L.vector(c + "in", hp.streams)) || !(W.hc_out[q] = L.vector(c + "out", hp.streams)) ||
-                    !(W.hc_mix[q] = L.vector2(c + "mix", hp.streams, hp.streams))) return false;
+                if (!((q ? W.norm2 : W.norm1) = L.vector(p + (q ? "norm2" : "norm1"), width))) return false;
+                if (hp.streams > 0 && (!(W.hc_in[q] = L.vector(c + "in", hp.streams)) || !(W.hc_out[q] = L.vector(c + "out", hp.streams)) || !(W.hc_mix[q] = L.vector2(c + "mix", hp.streams, hp.streams)))) return false;
             }
             const int64_t hd = (int64_t) H.heads * H.dim, hv = (int64_t) H.heads * H.vdim;
             if (H.mixer == PI_MIXER_MEMORY) {
@@ -481,22 +574,40 @@ bool llama_model::ensure_loaded_hybrid(int n_positions, std::string & err) {
                 if (!(W.gate_bias = L.vectors({ { m + "i.b", H.heads }, { m + "f.b", H.heads } }, 0)) || !(W.mix_norm = L.vector(m + "norm", hv))) return false;
             } else if (H.mixer == PI_MIXER_WINDOW_ATTENTION) {
                 const pi_gate_attention & A = H.left;
-                std::vector<std::pair<std::string, int64_t>> rows = { { m + "q", hd } }, biases = { { m + "q.b", hd } };
+                const int64_t qd = A.maps * hd;
+                std::vector<std::pair<std::string, int64_t>> rows = { { m + "q", qd } }, biases = { { m + "q.b", qd } };
                 if (H.kv_from < 0) {
-                    const int64_t gd = (int64_t) A.kv_heads * A.dim, gv = (int64_t) A.kv_heads * A.vdim;
+                    const int64_t gd = (int64_t) A.kv_heads * A.maps * A.dim, gv = (int64_t) A.kv_heads * A.vdim;
                     rows.push_back({ m + "k", gd }); rows.push_back({ m + "v", gv }); biases.push_back({ m + "k.b", gd }); biases.push_back({ m + "v.b", gv });
                 }
                 if (!(W.w_in = L.matrix(rows, width)) || (A.bias && !(W.in_bias = L.vectors(biases, 0)))) return false;
+                if (A.conv > 0) {
+                    std::vector<std::pair<std::string, int64_t>> taps;
+                    for (const auto & r : rows) taps.push_back({ r.first + ".conv", r.second });
+                    if (!(W.conv_w = L.vectors(taps, A.conv))) return false;
+                }
+                if (A.maps == 2) {
+                    std::vector<double> a, b; double e[2];
+                    for (int k = 0; k < 2; k++) {
+                        const std::string n = std::to_string(k + 1);
+                        if (!L.host_vector(m + "lq" + n, A.dim, a) || !L.host_vector(m + "lk" + n, A.dim, b)) return false;
+                        double dot = 0.0;
+                        for (int j = 0; j < A.dim; j++) dot += a[(size_t) j] * b[(size_t) j];
+                        e[k] = std::exp(dot);
+                    }
+                    W.lam = (float) (e[0] - e[1] + (double) A.diff);
+                }
             } else if (H.mixer == PI_MIXER_LATENT_ATTENTION) {
                 const pi_latent & A = H.latent;
                 std::vector<std::pair<std::string, int64_t>> rows = { { m + "dq", A.q_rank }, { m + "dkv", (int64_t) H.kv_rank + A.rot_dim } };
-                if (A.gated) rows.push_back({ m + "g", H.heads });
+                if (A.gated) rows.push_back({ m + "g", (int64_t) H.heads * A.gate_width });
+                if (A.sink && !(W.sink = L.vector(m + "sink", H.heads))) return false;
                 if (!(W.w_in = L.matrix(rows, width)) || !(W.q_norm = L.vector(m + "dq.norm", A.q_rank)) || !(W.mix_norm = L.vector(m + "dkv.norm", H.kv_rank))) return false;
                 if (!(W.w_uq = L.matrix({ { m + "uq", (int64_t) H.heads * (H.dim + A.rot_dim) } }, A.q_rank)) || !(W.w_uk = L.matrix({ { m + "uk", hd } }, H.kv_rank)) || !(W.w_uv = L.matrix({ { m + "uv", hv } }, H.kv_rank))) return false;
-            } else { err = "a block over residual streams has no mixer of kind " + std::to_string((int) H.mixer); return false; }
+            } else { err = "this kind of block has no mixer of kind " + std::to_string((int) H.mixer); return false; }
             if (H.mixer != PI_MIXER_MEMORY && !(W.rotary = rotary_of(H, std::max(n_positions, 32)))) { err = std::string("rotation table: ") + pi_last_error(); return false; }
             if (!(W.w_o = L.matrix({ { m + "o", width } }, hv))) return false;
-            if (H.mlp == PI_MLP_DENSE_SWIGLU && (!(W.ff_up = L.matrix({ { p + "mlp.gate", H.ff }, { p + "mlp.up", H.ff } }, width)) || !(W.ff_down = L.matrix({ { p + "mlp.down", width } }, H.ff)))) return false;
+            if ((H.mlp == PI_MLP_DENSE_SWIGLU || H.mlp == PI_MLP_DENSE_CLIPPED) && (!(W.ff_up = L.matrix({ { p + "mlp.gate", H.ff }, { p + "mlp.up", H.ff } }, width)) || !(W.ff_down = L.matrix({ { p + "mlp.down", width } }, H.ff)))) return false;
             W.loaded = true;
             continue;
         }
@@ -649,19 +760,20 @@ llama_model * load_hybrid_model(const std::string & folder, const llama_model_pa
     else if (arch->str == "Rafusun") hp.arch = PI_ARCH_RAFUSUN;
     else if (arch->str == "Rarevik") hp.arch = PI_ARCH_RAREVIK;
     else if (arch->str == "Rerizen") hp.arch = PI_ARCH_RERIZEN;
-    else return fail("architecture '" + arch->str + "' is not one this engine builds (Fasovik, Vikarax, Rafusun, Rarevik, Rerizen)");
+    else if (arch->str == "Letevik") hp.arch = PI_ARCH_LETEVIK;
+    else return fail("architecture '" + arch->str + "' is not one this engine builds (Fasovik, Vikarax, Rafusun, Rarevik, Rerizen, Letevik)");
     m->name = arch->str;
     double d;
     if (!int_at(cfg, "vocab", hp.n_vocab) || !int_at(cfg, "width", hp.n_embd) || hp.n_vocab < 1 || hp.n_embd < 1) return fail("'vocab' and 'width' must be positive integers");
-    if (hp.arch == PI_ARCH_VIKARAX || hp.arch == PI_ARCH_RAFUSUN || hp.arch == PI_ARCH_RAREVIK || hp.arch == PI_ARCH_RERIZEN) {
+    if (hp.arch != PI_ARCH_FASOVIK) {
         std::string what;
         if (!params.vocab_only && !m->st_file.open(folder + "/model.safetensors", err)) { fprintf(stderr, "llama_load_model_from_file: %s\n", err.c_str()); return nullptr; }
-        if (hp.arch == PI_ARCH_RERIZEN ? !read_rerizen_config(cfg, hp, what) : hp.arch == PI_ARCH_VIKARAX ? !read_vikarax_config(cfg, hp, what) : hp.arch == PI_ARCH_RAREVIK ? !read_rarevik_config(cfg, hp, what) : !read_rafusun_config(cfg, params.vocab_only ? nullptr : &m->st_file, hp, what)) return fail(what);
+        if (hp.arch == PI_ARCH_LETEVIK ? !read_letevik_config(cfg, hp, what) : hp.arch == PI_ARCH_RERIZEN ? !read_rerizen_config(cfg, hp, what) : hp.arch == PI_ARCH_VIKARAX ? !read_vikarax_config(cfg, hp, what) : hp.arch == PI_ARCH_RAREVIK ? !read_rarevik_config(cfg, hp, what) : !read_rafusun_config(cfg, params.vocab_only ? nullptr : &m->st_file, hp, what)) return fail(what);
         m->hweights.resize((size_t) hp.n_layer);
         if (!params.vocab_only) {
             for (const auto & kv : m->st_file.tensors) { m->n_elements += (uint64_t) kv.second.elements(); m->n_bytes += kv.second.nbytes; }
             const st_tensor * e = m->st_file.tensor("embed"), * h = m->st_file.tensor("head");
-            if (!e || e->shape != std::vector<int64_t>{ hp.n_vocab, hp.n_embd } || (hp.arch != PI_ARCH_RAREVIK && (!h || h->shape != e->shape))) return fail("tensors 'embed' and 'head' are missing or not [vocab][width]");
+            if (!e || e->shape != std::vector<int64_t>{ hp.n_vocab, hp.n_embd } || (hp.own_head && (!h || h->shape != e->shape))) return fail("tensors 'embed' and 'head' are missing or not [vocab][width]");
         }
         return m.release();
     }

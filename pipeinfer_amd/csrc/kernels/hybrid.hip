@@ -742,9 +742,9 @@ static lat_plan latent_plan(int heads, int rank, int rot, int n_tok, int n_ctx) 
 }
 
 // grid (token tile of 4, head, 64 values of the rank, then 64 values of the rotated part): lane = one rank value, the four waves take a quarter of the head's dim each and meet in LDS.  A query head is
-// [dim values | rot values]; the last are turned in neighbouring pairs by the token's position (cs: the rotation table) and go behind the rank values
+// [dim values | rot values]; the last are turned in pairs by the token's position (cs: the rotation table) and go behind the rank values
 __global__ void __launch_bounds__(256) k_latent_absorb(const float * __restrict__ q, int64_t qs, const uint16_t * __restrict__ wuk, float scale, int heads, int dim, int rank, int rot, const float2 * __restrict__ cs, int n_pos,
-                                                       const int32_t * __restrict__ pos, int n_tok, float * __restrict__ qa, const int32_t * __restrict__ abort_w) {
+                                                       int pairing, const int32_t * __restrict__ pos, int n_tok, float * __restrict__ qa, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 5)) return;
     __shared__ float part[4][4][64];
     extern __shared__ float4 qsh[];                                    // [dim]: the head's query values of the four tokens, side by side
@@ -754,9 +754,10 @@ __global__ void __launch_bounds__(256) k_latent_absorb(const float * __restrict_
         const int d = (blockIdx.z - n_rank_blocks) * 64 + lane, t = t0 + wave;
         if (d >= rot || t >= n_tok) return;
         const float * qr = q + (int64_t) t * qs + (int64_t) h * hw + dim;
-        const float2 c = cs[(int64_t) min(pos[t], n_pos - 1) * (rot / 2) + (d >> 1)];
-        const float own = qr[d], other = qr[d ^ 1];
-        qa[((int64_t) t * heads + h) * (rank + rot) + rank + d] = ((d & 1) ? own * c.x + other * c.y : own * c.x - other * c.y) * scale;
+        const pi_turn u = pi_turn_of(d, rot / 2, pairing);
+        const float2 c = cs[(int64_t) min(pos[t], n_pos - 1) * (rot / 2) + u.angle];
+        const float own = qr[d], other = qr[u.mate];
+        qa[((int64_t) t * heads + h) * (rank + rot) + rank + d] = (u.lead ? own * c.x - other * c.y : own * c.x + other * c.y) * scale;
         return;
     }
     for (int idx = threadIdx.x; idx < 4 * dim; idx += 256) {
@@ -939,21 +940,22 @@ __global__ void __launch_bounds__(256) k_latent_scores(const float * __restrict_
     }
 }
 
-// grid (token tile of 4, head, 16 output values): merges the splits (with the sink if there is one), normalises, applies its rows of W_uv[h], then the head's gate if there is one
+// grid (token tile of 4, head, 16 output values): merges the splits (with the sink if there is one), normalises, applies its rows of W_uv[h], then the gate if there is one: one value per head, or (gate_width = vdim)
+// one per output value
 __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict__ pol, const float * __restrict__ pml, const uint16_t * __restrict__ wuv, const float * __restrict__ sink,
-                                                        const float * __restrict__ gate, int64_t gs, int gate_act, int heads, int vdim, int rank, int S, int n_tok, float * __restrict__ out, int64_t os,
+                                                        const float * __restrict__ gate, int64_t gs, int gate_act, int gate_width, int heads, int vdim, int rank, int S, int n_tok, float * __restrict__ out, int64_t os,
                                                         const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 5)) return;
     extern __shared__ float ol[];                                     // [4][rank]
     __shared__ float wgt[4][64];                                      // per token: weight of the splits that hold something, 64 splits at a time,
     __shared__ int num[4][64], cnt[4];                                // their numbers, how many they are
-    __shared__ float gsh[4];                                          // per token: the head's gate
+    __shared__ float gsh[4];                                          // per token: the head's gate (one value per head)
     const int t0 = blockIdx.x * 4, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int nt = min(4, n_tok - t0);
     for (int idx = tid; idx < 4 * rank; idx += 256) ol[idx] = 0.0f;
     if (tid < 4) {
         float g = 1.0f;
-        if (gate && tid < nt) { g = gate[(int64_t) (t0 + tid) * gs + h]; if (gate_act == PI_ACT_SIGMOID) g = 1.0f / (1.0f + expf(-g)); }
+        if (gate && gate_width == 1 && tid < nt) { g = gate[(int64_t) (t0 + tid) * gs + h]; if (gate_act == PI_ACT_SIGMOID) g = 1.0f / (1.0f + expf(-g)); }
         gsh[tid] = g;
     }
     // (the wave `tt` owns token t0 + tt's bookkeeping)
@@ -1001,7 +1003,11 @@ __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict
 #pragma unroll
         for (int tt = 0; tt < 4; tt++) {
             const float v = pi_lanes_sum<64>(a[tt]);
-            if (lane == 0 && tt < nt) out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v * gsh[tt];
+            if (lane == 0 && tt < nt) {
+                float g = gsh[tt];
+                if (gate && gate_width > 1) { g = gate[(int64_t) (t0 + tt) * gs + (int64_t) h * vdim + vv]; if (gate_act == PI_ACT_SIGMOID) g = 1.0f / (1.0f + expf(-g)); }
+                out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v * g;
+            }
         }
     }
 }
@@ -1038,6 +1044,12 @@ extern "C" int pi_op_latent_attention(const float * q, int64_t q_stride, const f
 extern "C" int pi_op_latent_attention_rot(const float * q, int64_t q_stride, const float * cache, const uint32_t * mask, const pi_weight * wuk, const pi_weight * wuv, const float * sink_dev, const float * gate_dev,
                                           int64_t gate_stride, int gate_act, float scale, int heads, int dim, int rot, int vdim, int rank, const void * rotary_table, const int32_t * pos_dev, int n_tok, int n_kv,
                                           float * scratch_dev, size_t scratch_floats, float * out, int64_t out_stride, const int32_t * dyn_dev, void * stream) {
+    return pi_op_latent_attention_gated(q, q_stride, cache, mask, wuk, wuv, sink_dev, gate_dev, gate_stride, gate_act, 1, scale, heads, dim, rot, vdim, rank, rotary_table, PI_PAIR_NEIGHBOURS, pos_dev, n_tok, n_kv, scratch_dev,
+                                        scratch_floats, out, out_stride, dyn_dev, stream);
+}
+extern "C" int pi_op_latent_attention_gated(const float * q, int64_t q_stride, const float * cache, const uint32_t * mask, const pi_weight * wuk, const pi_weight * wuv, const float * sink_dev, const float * gate_dev,
+                                            int64_t gate_stride, int gate_act, int gate_width, float scale, int heads, int dim, int rot, int vdim, int rank, const void * rotary_table, int pairing, const int32_t * pos_dev,
+                                            int n_tok, int n_kv, float * scratch_dev, size_t scratch_floats, float * out, int64_t out_stride, const int32_t * dyn_dev, void * stream) {
     if (n_tok <= 0) return 0;
     const float2 * cs = nullptr; int n_pos = 0, half = 0;
     if (rot < 0 || (rot & 1)) { pi_set_error("pi_op_latent_attention: %d rotated dimensions (an even number)", rot); return -1; }
@@ -1045,7 +1057,9 @@ extern "C" int pi_op_latent_attention_rot(const float * q, int64_t q_stride, con
         pi_rotary_table_view(rotary_table, &cs, &n_pos, &half);
         if (!cs || half != rot / 2 || !pos_dev) { pi_set_error("pi_op_latent_attention: a rotation table over the %d rotated dimensions and the tokens' positions are required", rot); return -1; }
     }
+    if (pairing != PI_PAIR_HALVES && pairing != PI_PAIR_NEIGHBOURS) { pi_set_error("pi_op_latent_attention: pairing %d is unknown", pairing); return -1; }
     if (gate_dev && gate_act != PI_ACT_NONE && gate_act != PI_ACT_SIGMOID) { pi_set_error("pi_op_latent_attention: gate activation %d is unknown", gate_act); return -1; }
+    if (gate_dev && gate_width != 1 && gate_width != vdim) { pi_set_error("pi_op_latent_attention: a gate has one value per head or one per output value (%d), not %d", vdim, gate_width); return -1; }
     if (q_stride < (int64_t) heads * (dim + rot)) { pi_set_error("pi_op_latent_attention: query rows of %lld floats hold no %d heads of %d + %d values", (long long) q_stride, heads, dim, rot); return -1; }
     if (!wuk || !wuv || wuk->type != PI_BF16 || wuv->type != PI_BF16 || wuk->ne0 != rank || wuv->ne0 != rank || wuk->ne1 != (int64_t) heads * dim || wuv->ne1 != (int64_t) heads * vdim) {
         pi_set_error("pi_op_latent_attention: the up-projections must be bfloat16 [heads * dim][rank] and [heads * vdim][rank]"); return -1;
@@ -1060,7 +1074,7 @@ extern "C" int pi_op_latent_attention_rot(const float * q, int64_t q_stride, con
     const int nta = std::min(n_tok, PI_KT_MAXNT - 1);
     const int acct = pi_account_n_kv() > 0 ? pi_account_n_kv() : n_kv;
     PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, 2.0 * rank * heads * dim + 4.0 * n_tok * heads * (dim + rank + 2.0 * rot), k_latent_absorb, dim3((unsigned) ((n_tok + 3) / 4), (unsigned) heads, (unsigned) ((rank + 63) / 64 + (rot + 63) / 64)), dim3(256), (size_t) 16 * dim, s,
-                 q, q_stride, (const uint16_t *) wuk->p0, scale, heads, dim, rank, rot, cs, n_pos, pos_dev, n_tok, qa, pi_abort_word());
+                 q, q_stride, (const uint16_t *) wuk->p0, scale, heads, dim, rank, rot, cs, n_pos, pairing, pos_dev, n_tok, qa, pi_abort_word());
     PI_CHECK_LAUNCH();
     const dim3 grid((unsigned) n_tok, (unsigned) ((heads + p.M - 1) / p.M), (unsigned) p.S);
     const double bytes = 4.0 * acct * (rank + rot) + 4.0 * n_tok * heads * (rank + rot + (double) rank * p.S);
@@ -1071,7 +1085,7 @@ extern "C" int pi_op_latent_attention_rot(const float * q, int64_t q_stride, con
 #undef LAT_GO
     PI_CHECK_LAUNCH();
     PI_KT_LAUNCH(PI_KT_ATT, PI_BF16, nta, 2.0 * rank * heads * vdim + 4.0 * n_tok * heads * (rank * p.S + vdim), k_latent_combine, dim3((unsigned) ((n_tok + 3) / 4), (unsigned) heads, (unsigned) ((vdim + 15) / 16)), dim3(256), (size_t) 16 * rank, s,
-                 pol, pml, (const uint16_t *) wuv->p0, sink_dev, gate_dev, gate_stride, gate_act, heads, vdim, rank, p.S, n_tok, out, out_stride, pi_abort_word());
+                 pol, pml, (const uint16_t *) wuv->p0, sink_dev, gate_dev, gate_stride, gate_act, gate_width, heads, vdim, rank, p.S, n_tok, out, out_stride, pi_abort_word());
     PI_CHECK_LAUNCH(); return 0;
 }
 

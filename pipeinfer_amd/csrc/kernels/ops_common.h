@@ -47,6 +47,12 @@ int pi_account_n_kv();                                       // > 0: the cells a
 int pi_cu_count();
 const pi_tables & pi_get_tables();
 void pi_rotary_table_view(const void * table, const float2 ** cs, int * n_pos, int * half);      // a rotation table's device rows [n_pos][half] of (cos, sin) (nothing for a null table)
+// dimension i of a rotated vector of 2 * half values: its mate, the number of its angle, whether it is the pair's first member (u cos - v sin; the second: v cos + u sin)
+struct pi_turn { int mate, angle; bool lead; };
+static __device__ __forceinline__ pi_turn pi_turn_of(int i, int half, int pairing) {
+    if (pairing == PI_PAIR_NEIGHBOURS) return { i ^ 1, i >> 1, (i & 1) == 0 };
+    return i < half ? pi_turn{ i + half, i, true } : pi_turn{ i - half, i - half, false };
+}
 
 #define PI_CHECK_HIP(expr)                                                                   \
     do {                                                                                     \

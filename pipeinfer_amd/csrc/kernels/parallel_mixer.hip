@@ -5,6 +5,7 @@
 //
 //   k_qkv_prepare        per token: RMS norm (shared per-head weight) + partial rotation of q and k, unit RMS of v; k and v go to the token's cache cell, the cell learns its position
 //   k_chunk_attention    out[t][h] = gate[t][h] * sum over visible cells c of sigmoid(q . K[c] * scale + bias[h]) V[c];  visible = the pass's mask bit AND position(c) >= start of t's chunk
+//                        (two maps per head: both maps' soft-max outputs over the same values, the second subtracted with a factor, the difference RMS-normed)
 //   k_causal_conv        per channel: act(bias + sum_l w[l] * input(t - taps + 1 + l)), inputs before the pass come from the sequence's conv state (zeros for a fresh one)
 //   k_conv_state_update  the sequence's last taps - 1 inputs, for the next pass
 //   k_causal_conv_walk   both of the above and k_ssd_steps in one launch for passes of at most 32 tokens
@@ -160,9 +161,9 @@ extern "C" int pi_op_qkv_prepare(const float * q, const float * k, const float *
 }
 
 // the same with the order and the pairing as parameters.  norm_first: R(.) * w, then the rotation (as above), else the rotation first and R(.) * w over the rotated head; w may be absent (1);
-// pairing PI_PAIR_HALVES: dimension i with i + dims / 2, PI_PAIR_NEIGHBOURS: 2i with 2i + 1 (angle number i either way); v_norm = 0: value heads go to their cell as they are
+// pairing PI_PAIR_HALVES: dimension i with i + dims / 2, PI_PAIR_NEIGHBOURS: 2i with 2i + 1 (angle number i either way); v_norm = 0: value heads go to their cell as they are.  G key heads, GV value heads
 __global__ void __launch_bounds__(64) k_qkv_prepare_any(const float * __restrict__ q, const float * __restrict__ k, const float * __restrict__ v, int64_t stride, const float * __restrict__ qw,
-                                                        const float * __restrict__ kw, float eps, int H, int G, int D, int V, const float2 * __restrict__ rot, int half, int n_pos, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every,
+                                                        const float * __restrict__ kw, float eps, int H, int G, int GV, int D, int V, const float2 * __restrict__ rot, int half, int n_pos, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every,
                                                         const int32_t * __restrict__ pos, float * __restrict__ q_out, int64_t qos, float * __restrict__ kc, float * __restrict__ vc,
                                                         int32_t * __restrict__ cell_pos, const int32_t * __restrict__ dyn, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w)) return;
@@ -179,7 +180,7 @@ __global__ void __launch_bounds__(64) k_qkv_prepare_any(const float * __restrict
             for (int i = lane; i < V; i += 64) ss = fmaf(src[i], src[i], ss);
             inv = 1.0f / sqrtf(pi_lanes_sum<64>(ss) / (float) V + eps);
         }
-        float * dst = vc + ((int64_t) cell * G + g) * V;
+        float * dst = vc + ((int64_t) cell * GV + g) * V;
         for (int i = lane; i < V; i += 64) dst[i] = v_norm ? src[i] * inv : src[i];
         return;
     }
@@ -202,11 +203,10 @@ __global__ void __launch_bounds__(64) k_qkv_prepare_any(const float * __restrict
     auto turned = [&](int i) {
         float y = before(i);
         if (i < 2 * half) {
-            const bool lead = pairing == PI_PAIR_NEIGHBOURS ? !(i & 1) : i < half;                       // the pair's first member: u cos - v sin; its second: v cos + u sin
-            const int j = pairing == PI_PAIR_NEIGHBOURS ? (i ^ 1) : (i < half ? i + half : i - half), f = pairing == PI_PAIR_NEIGHBOURS ? (i >> 1) : (i < half ? i : i - half);
-            const float o = before(j);
-            const float2 c = cs[f];
-            y = lead ? y * c.x - o * c.y : y * c.x + o * c.y;
+            const pi_turn u = pi_turn_of(i, half, pairing);
+            const float o = before(u.mate);
+            const float2 c = cs[u.angle];
+            y = u.lead ? y * c.x - o * c.y : y * c.x + o * c.y;
         }
         return y;
     };
@@ -222,9 +222,9 @@ extern "C" int pi_op_qkv_prepare_ex(const float * q, const float * k, const floa
     if (n_tok > 0 && (!k || !v)) { pi_set_error("pi_op_qkv_prepare: keys and values are required"); return -1; }
     return pi_op_qkv_prepare_temp(q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, dim, vdim, rotary_table, norm_first, pairing, v_norm, 0.0f, 0, pos_dev, n_tok, q_out, q_out_stride, k_cache, v_cache, cell_pos_dev, dyn_dev, stream);
 }
-extern "C" int pi_op_qkv_prepare_temp(const float * q, const float * k, const float * v, int64_t stride, const float * q_norm_w, const float * k_norm_w, float eps, int heads, int kv_heads, int dim, int vdim,
-                                      const void * rotary_table, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every, const int32_t * pos_dev, int n_tok, float * q_out, int64_t q_out_stride,
-                                      float * k_cache, float * v_cache, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream) {
+static int qkv_prepare(const float * q, const float * k, const float * v, int64_t stride, const float * q_norm_w, const float * k_norm_w, float eps, int heads, int kv_heads, int value_heads, int dim, int vdim,
+                       const void * rotary_table, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every, const int32_t * pos_dev, int n_tok, float * q_out, int64_t q_out_stride,
+                       float * k_cache, float * v_cache, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream) {
     if (n_tok <= 0) return 0;
     const pi_rotary_table * rt = (const pi_rotary_table *) rotary_table;
     if (!rt || 2 * rt->half > dim) { pi_set_error("pi_op_qkv_prepare: a rotation table over at most %d dimensions is required", dim); return -1; }
@@ -234,15 +234,31 @@ extern "C" int pi_op_qkv_prepare_temp(const float * q, const float * k, const fl
     if (pairing != PI_PAIR_HALVES && pairing != PI_PAIR_NEIGHBOURS) { pi_set_error("pi_op_qkv_prepare: pairing %d is unknown", pairing); return -1; }
     if (norm_first < 0 || norm_first > PI_QK_NORM_NONE) { pi_set_error("pi_op_qkv_prepare: norm order %d is unknown", norm_first); return -1; }
     if (norm_first == PI_QK_NORM_FIRST && (!q_norm_w || !k_norm_w)) { pi_set_error("pi_op_qkv_prepare: norm weights are required"); return -1; }
-    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 8.0 * n_tok * ((double) heads * dim + (double) kv_heads * (dim + vdim)), k_qkv_prepare_any, dim3((unsigned) n_tok, (unsigned) (heads + (k ? 2 * kv_heads : 0))), dim3(64), 0, (hipStream_t) stream,
-                 q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, dim, vdim, rt->cs, rt->half, rt->n_pos, norm_first, pairing, v_norm, temp_coef, temp_every, pos_dev, q_out, q_out_stride, k_cache, v_cache, cell_pos_dev, dyn_dev, pi_abort_word());
+    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 8.0 * n_tok * ((double) (heads + kv_heads) * dim + (double) value_heads * vdim), k_qkv_prepare_any, dim3((unsigned) n_tok, (unsigned) (heads + (k ? kv_heads + value_heads : 0))), dim3(64), 0, (hipStream_t) stream,
+                 q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, value_heads, dim, vdim, rt->cs, rt->half, rt->n_pos, norm_first, pairing, v_norm, temp_coef, temp_every, pos_dev, q_out, q_out_stride, k_cache, v_cache, cell_pos_dev, dyn_dev,
+                 pi_abort_word());
     PI_CHECK_LAUNCH(); return 0;
+}
+extern "C" int pi_op_qkv_prepare_temp(const float * q, const float * k, const float * v, int64_t stride, const float * q_norm_w, const float * k_norm_w, float eps, int heads, int kv_heads, int dim, int vdim,
+                                      const void * rotary_table, int norm_first, int pairing, int v_norm, float temp_coef, int temp_every, const int32_t * pos_dev, int n_tok, float * q_out, int64_t q_out_stride,
+                                      float * k_cache, float * v_cache, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream) {
+    return qkv_prepare(q, k, v, stride, q_norm_w, k_norm_w, eps, heads, kv_heads, kv_heads, dim, vdim, rotary_table, norm_first, pairing, v_norm, temp_coef, temp_every, pos_dev, n_tok, q_out, q_out_stride, k_cache, v_cache,
+                       cell_pos_dev, dyn_dev, stream);
+}
+// heads of `maps` query / key maps over one value: every map is a head of its own here, without norms
+extern "C" int pi_op_qkv_prepare_maps(const float * q, const float * k, const float * v, int64_t stride, int heads, int kv_heads, int maps, int dim, int vdim, const void * rotary_table, int pairing, const int32_t * pos_dev, int n_tok,
+                                      float * q_out, int64_t q_out_stride, float * k_cache, float * v_cache, int32_t * cell_pos_dev, const int32_t * dyn_dev, void * stream) {
+    if (n_tok > 0 && (!k || !v || maps < 1)) { pi_set_error("pi_op_qkv_prepare: keys, values and at least one map are required"); return -1; }
+    return qkv_prepare(q, k, v, stride, nullptr, nullptr, 0.0f, heads * maps, kv_heads * maps, kv_heads, dim, vdim, rotary_table, PI_QK_NORM_NONE, pairing, 0, 0.0f, 0, pos_dev, n_tok, q_out, q_out_stride, k_cache, v_cache,
+                       cell_pos_dev, dyn_dev, stream);
 }
 
 // ---- attention with sigmoid weights inside chunks ---------------------------------------------------------------------------------------------------------
 // grid (token, key / value head, split of its query heads): the workgroup serves the query heads of its key head (all of them in one workgroup unless they are very many or very wide).  The cells are walked 256 at a time; the visible ones of a round are compacted
 // in cell order (so that the sum has one order whatever the launch), their key rows staged in LDS 64 at a time.  Scores: thread (cell, query head); output: thread (query
 // head, value column), value rows read from the cache along the columns.
+// MAPS = 2: a query / key head is two maps of D values each over ONE value row; the workgroup serves 2 * hpg rows (head, map) from the same key and value tiles, and ends with
+// R(a1 - lam a2) * out_mult per head (R: divided by the root mean square over the head's V values)
 // rows `cells[0 .. nl)` of a cache [cells][G][W] (head g) into LDS rows `pitch` floats apart.  Eight loads per thread are issued before the first LDS store: the compiler cannot
 // tell the cell list (LDS) from the tile (LDS) and would otherwise wait for every row's trip to memory before it reads the next cell number
 // RPW: rows a wave has in flight per round
@@ -286,11 +302,20 @@ static __device__ __forceinline__ void ca_stage(const float * __restrict__ cache
 #define CA_TILE 64                                // key rows staged at a time (fewer when a row is long: ca_tile)
 #define CA_SB 1                                   // blocks of 256 cells whose visibility is worked out in one round
 #define CA_MAXOUT 16                              // outputs (query head, value column) a thread accumulates: hpg * vdim <= 256 * CA_MAXOUT
-template <int RPW>
+// how the two maps of a head meet: lam, and the epsilon of the norm over their difference
+struct ca_maps { float lam, eps; };
+// the difference of a head's two map outputs a1[V], a2[V] (already divided by their denominators), normed; one wave
+static __device__ __forceinline__ void ca_join_maps(const float * a1, const float * a2, int V, ca_maps mp, float out_mult, float * __restrict__ out, int lane) {
+    float ss = 0.0f;
+    for (int v = lane; v < V; v += 64) { const float o = a1[v] - mp.lam * a2[v]; ss = fmaf(o, o, ss); }
+    const float inv = out_mult / sqrtf(pi_lanes_sum<64>(ss) / (float) V + mp.eps);
+    for (int v = lane; v < V; v += 64) out[v] = (a1[v] - mp.lam * a2[v]) * inv;
+}
+template <int RPW, int MAPS>
 __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restrict__ q, int64_t qs, const float * kc, const float * vc, const int32_t * __restrict__ cell_pos,
                                                          const uint32_t * __restrict__ mask, const int32_t * __restrict__ pos, const float * __restrict__ hbias, const float * __restrict__ gate, int64_t gs, int gate_act,
                                                          float scale, float out_mult, int weights, float softcap, int chunk, int H, int G, int D, int V, int n_kv_arg, int tile, int hps, float * __restrict__ out, int64_t os, const int32_t * __restrict__ dyn,
-                                                         const float * __restrict__ sink, int mask_kind, int pool, int pool_off, int pool_z, int n_hz, int n_cs, int split_cells, float * __restrict__ part, const int32_t * __restrict__ abort_w) {
+                                                         const float * __restrict__ sink, int mask_kind, int pool, int pool_off, int pool_z, int n_hz, int n_cs, int split_cells, float * __restrict__ part, int keep_first, ca_maps mp, const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w, 5)) return;
     extern __shared__ float lds[];                // q [hpg][D] | key tile [tile][D + 1], then the value tile [tile][V] in the same place | weights [tile][hpg]
     if (pool_z > 0 && (int) blockIdx.z == pool_z) {                   // the extra slice of workgroups: the pooled rows of the blocks this pass's tokens close (no token of the pass reads them: the host checked n_tok <= window)
@@ -304,14 +329,15 @@ __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restric
     // blockIdx.z = head split + n_hz * cell split.  split_cells > 0 (soft-max kinds, few tokens): this workgroup looks at the cells [cs * split_cells, (cs + 1) * split_cells) only and leaves its running
     // maximum, denominator and un-normalised sums in `part` for k_attention_combine: a single token's tiles then run side by side instead of one after the other
     const int hz = (int) blockIdx.z % n_hz, cs = (int) blockIdx.z / n_hz;
-    const int hs = hz * hps, hpg = min(hps, H / G - hs), h0 = g * (H / G) + hs, DP = D + 1;        // this workgroup's query heads: hpg of them from h0 on (all of the key head's unless they are split over blockIdx.z)
-    float * qsh = lds, * ksh = qsh + hpg * D, * wsh = ksh + tile * max(DP, V);
-    float * m_run = wsh + tile * hps, * l_run = m_run + hps, * f_run = l_run + hps;        // soft-max weights: per query head the running maximum, denominator, and the factor the sums so far take this tile
+    const int hs = hz * hps, hpg = min(hps, H / G - hs), h0 = g * (H / G) + hs, KD = MAPS * D, DP = KD + 1;        // this workgroup's query heads: hpg of them from h0 on (all of the key head's unless they are split over blockIdx.z)
+    const int nr = MAPS * hpg, nrs = MAPS * hps;          // its rows of scores: (head, map)
+    float * qsh = lds, * ksh = qsh + nr * D, * wsh = ksh + tile * max(DP, V);
+    float * m_run = wsh + tile * nrs, * l_run = m_run + nrs, * f_run = l_run + nrs;        // soft-max weights: per query head the running maximum, denominator, and the factor the sums so far take this tile
     const bool soft = weights != PI_WEIGHTS_SIGMOID;
     // (a sink: one more key without a value, of score 0 or of a learned score per head that the scale does not touch)
-    if (soft) for (int m = tid; m < hpg; m += 256) {
+    if (soft) for (int m = tid; m < nr; m += 256) {
         const bool has_sink = split_cells == 0 && (sink || weights == PI_WEIGHTS_SOFTMAX_SINK);           // (with cell splits the sink joins in the combine)
-        m_run[m] = has_sink ? (sink ? sink[h0 + m] : 0.0f) : -INFINITY; l_run[m] = has_sink ? 1.0f : 0.0f;
+        m_run[m] = has_sink ? (sink ? sink[h0 + m / MAPS] : 0.0f) : -INFINITY; l_run[m] = has_sink ? 1.0f : 0.0f;
     }
     const int n_kv = min(dyn ? dyn[1] : n_kv_arg, n_kv_arg);
     const int words = (n_kv_arg + 31) / 32;
@@ -319,11 +345,11 @@ __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restric
     const int p = pos[t];
     // the first position the token sees as itself: the start of its block of `chunk` positions, or of the window of `chunk` positions that ends with the token
     const int first_pos = chunk <= 0 ? 0 : mask_kind == PI_MASK_WINDOW ? p - chunk + 1 : p / chunk * chunk;
-    for (int i = tid; i < hpg * D; i += 256) qsh[i] = q[(int64_t) t * qs + (int64_t) h0 * D + i];
+    for (int i = tid; i < nr * D; i += 256) qsh[i] = q[(int64_t) t * qs + (int64_t) h0 * KD + i];
     float acc[CA_MAXOUT];
 #pragma unroll
     for (int i = 0; i < CA_MAXOUT; i++) acc[i] = 0.0f;
-    const int n_out = hpg * V;
+    const int n_out = nr * V;
     const int c_first = split_cells > 0 ? cs * split_cells : 0, c_end = split_cells > 0 ? min(n_kv, c_first + split_cells) : n_kv;
     for (int c0 = c_first; c0 < c_end; c0 += 256 * CA_SB) {          // CA_SB blocks of 256 cells at a time: their mask words and positions are loaded together
         bool vis[CA_SB], far[CA_SB]; unsigned long long bal[CA_SB];
@@ -335,7 +361,7 @@ __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restric
             const int cp = in ? cell_pos[c] : -1;
             // behind the window a cell counts where it closes a block of `pool` positions, through the block's pooled row (row pool_off + cell of both caches)
             far[u] = pool > 0 && cp < first_pos && cp >= 0 && (cp + 1) % pool == 0;
-            vis[u] = in && ((word >> (c & 31)) & 1u) && (cp >= first_pos || far[u]);
+            vis[u] = in && ((word >> (c & 31)) & 1u) && (cp >= first_pos || far[u] || cp < keep_first);
         }
 #pragma unroll
         for (int u = 0; u < CA_SB; u++) bal[u] = __ballot(vis[u]);
@@ -356,25 +382,25 @@ __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restric
         for (int l0 = 0; l0 < total; l0 += tile) {
             const int nl = min(tile, total - l0);
             if (l0) __syncthreads();                 // (the previous tile's values are no longer read)
-            ca_stage<RPW>(kc, list + l0, nl, G, g, D, DP, ksh, tid);
+            ca_stage<RPW>(kc, list + l0, nl, G, g, KD, DP, ksh, tid);
             __syncthreads();
-            for (int i = tid; i < nl * hpg; i += 256) {
+            for (int i = tid; i < nl * nr; i += 256) {
                 const int cc = i % nl, m = i / nl;
-                const float * kr = ksh + cc * DP, * qr = qsh + m * D;
+                const float * kr = ksh + cc * DP + m % MAPS * D, * qr = qsh + m * D;
                 float s = 0.0f;
                 for (int d = 0; d < D; d++) s = fmaf(qr[d], kr[d], s);
-                s = s * scale + (hbias ? hbias[h0 + m] : 0.0f);
+                s = s * scale + (hbias ? hbias[h0 + m / MAPS] : 0.0f);
                 if (soft && softcap > 0.0f) s = softcap * tanhf(s / softcap);
-                wsh[cc * hpg + m] = soft ? s : pm_sigmoid(s);
+                wsh[cc * nr + m] = soft ? s : pm_sigmoid(s);
             }
             __syncthreads();
             if (soft)                             // a wave per query head, a lane per cell of the tile (tile <= 64): new maximum, exponentials in the scores' place, denominator
-                for (int m = wave; m < hpg; m += 4) {
-                    const float sc = lane < nl ? wsh[lane * hpg + m] : -INFINITY;
+                for (int m = wave; m < nr; m += 4) {
+                    const float sc = lane < nl ? wsh[lane * nr + m] : -INFINITY;
                     const float m_old = m_run[m], m_new = fmaxf(m_old, pi_wave_max(sc));
                     const float e = lane < nl ? expf(sc - m_new) : 0.0f;
                     const float sum = pi_lanes_sum<64>(e);
-                    if (lane < nl) wsh[lane * hpg + m] = e;
+                    if (lane < nl) wsh[lane * nr + m] = e;
                     if (lane == 0) { const float f = m_old == -INFINITY ? 0.0f : expf(m_old - m_new); m_run[m] = m_new; l_run[m] = fmaf(l_run[m], f, sum); f_run[m] = f; }
                 }
             // the value rows take the key tile's place: all their loads are in flight together (read one by one in the sum below, every row would cost a trip to memory)
@@ -386,7 +412,7 @@ __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restric
                 if (o < n_out) {
                     const int m = o / V, vv = o % V;
                     float a = soft ? acc[oi] * f_run[m] : acc[oi];
-                    for (int cc = 0; cc < nl; cc++) a = fmaf(wsh[cc * hpg + m], ksh[cc * V + vv], a);
+                    for (int cc = 0; cc < nl; cc++) a = fmaf(wsh[cc * nr + m], ksh[cc * V + vv], a);
                     acc[oi] = a;
                 }
             }
@@ -397,9 +423,20 @@ __global__ void __launch_bounds__(256) k_chunk_attention(const float * __restric
 #pragma unroll
         for (int oi = 0; oi < CA_MAXOUT; oi++) {
             const int o = oi * 256 + tid;
-            if (o < n_out) { const int m = o / V; part[(((int64_t) t * H + h0 + m) * n_cs + cs) * (V + 2) + o % V] = acc[oi]; }
+            if (o < n_out) { const int m = o / V; part[((((int64_t) t * H + h0) * MAPS + m) * n_cs + cs) * (V + 2) + o % V] = acc[oi]; }
         }
-        for (int m = tid; m < hpg; m += 256) { float * pr = part + (((int64_t) t * H + h0 + m) * n_cs + cs) * (V + 2) + V; pr[0] = m_run[m]; pr[1] = l_run[m]; }
+        for (int m = tid; m < nr; m += 256) { float * pr = part + ((((int64_t) t * H + h0) * MAPS + m) * n_cs + cs) * (V + 2) + V; pr[0] = m_run[m]; pr[1] = l_run[m]; }
+        return;
+    }
+    if constexpr (MAPS == 2) {                                        // both maps' outputs meet in LDS (over the queries and the tiles, which are no longer read), a wave per head
+        float den[CA_MAXOUT];
+#pragma unroll
+        for (int oi = 0; oi < CA_MAXOUT; oi++) { const int o = oi * 256 + tid; den[oi] = o < n_out ? l_run[o / V] : 0.0f; }
+        __syncthreads();
+#pragma unroll
+        for (int oi = 0; oi < CA_MAXOUT; oi++) { const int o = oi * 256 + tid; if (o < n_out) lds[o] = den[oi] > 0.0f ? acc[oi] / den[oi] : 0.0f; }
+        __syncthreads();
+        for (int m = wave; m < hpg; m += 4) ca_join_maps(lds + 2 * m * V, lds + (2 * m + 1) * V, V, mp, out_mult, out + (int64_t) t * os + (int64_t) (h0 + m) * V, lane);
         return;
     }
 #pragma unroll
@@ -435,6 +472,29 @@ __global__ void __launch_bounds__(128) k_attention_combine(const float * __restr
         out[(int64_t) t * os + (int64_t) h * V + v] = (den > 0.0f ? a / den : 0.0f) * gt * out_mult;
     }
 }
+// the same where a head is two maps: grid (token, head), both maps' splits merged into LDS, then joined by one wave
+__global__ void __launch_bounds__(128) k_attention_combine_maps(const float * __restrict__ part, int n_cs, int H, int V, ca_maps mp, float out_mult, float * __restrict__ out, int64_t os, const int32_t * __restrict__ abort_w) {
+    if (pi_aborted(abort_w)) return;
+    extern __shared__ float maps_lds[];                               // [2][V]
+    const int t = blockIdx.x, h = blockIdx.y, map = threadIdx.x >> 6, lane = threadIdx.x & 63;        // a wave per map
+    const float * pr = part + (((int64_t) t * H + h) * 2 + map) * n_cs * (V + 2);
+    // (the splits' maxima and denominators are read side by side, a lane per split: n_cs <= CA_SPLIT_MAX <= 64)
+    const float ms_l = lane < n_cs ? pr[(int64_t) lane * (V + 2) + V] : -INFINITY;
+    const float M = pi_wave_max(ms_l);
+    const float f_l = ms_l != -INFINITY ? expf(ms_l - M) : 0.0f;
+    const float den = pi_lanes_sum<64>(f_l > 0.0f ? pr[(int64_t) lane * (V + 2) + V + 1] * f_l : 0.0f);
+    for (int v0 = 0; v0 < V; v0 += 64) {
+        const int v = v0 + lane;
+        float a = 0.0f;
+        for (int s = 0; s < n_cs; s++) {
+            const float f = __shfl(f_l, s, 64);
+            if (f > 0.0f && v < V) a = fmaf(pr[(int64_t) s * (V + 2) + v], f, a);
+        }
+        if (v < V) maps_lds[map * V + v] = den > 0.0f ? a / den : 0.0f;
+    }
+    __syncthreads();
+    if (map == 0) ca_join_maps(maps_lds, maps_lds + V, V, mp, out_mult, out + (int64_t) t * os + (int64_t) h * V, lane);
+}
 // cell splits of a pass of n_tok tokens over n_kv cells: how many, and the floats of scratch they need (0 splits: the pass is wide enough to fill the device by itself)
 #define CA_SPLIT_MAX 32
 static int ca_cell_splits(int n_tok, int kv_heads, int n_hz, int n_kv, int * split_cells) {
@@ -457,12 +517,31 @@ extern "C" int pi_op_chunk_attention_ex(const float * q, int64_t q_stride, const
     return pi_op_window_attention(q, q_stride, (float *) k_cache, (float *) v_cache, cell_pos_dev, mask_dev, pos_dev, head_bias_dev, nullptr, gate_dev, gate_stride, gate_act, scale, out_mult, weights, softcap, PI_MASK_CHUNK, chunk, 0, 0, 0,
                                   heads, kv_heads, dim, vdim, n_tok, n_kv, nullptr, 0, out, out_stride, dyn_dev, stream);
 }
+static int window_attention(const float * q, int64_t q_stride, float * k_cache, float * v_cache, const int32_t * cell_pos_dev, const uint32_t * mask_dev, const int32_t * pos_dev, const float * head_bias_dev, const float * sink_dev,
+                            const float * gate_dev, int64_t gate_stride, int gate_act, float scale, float out_mult, int weights, float softcap, int mask_kind, int chunk, int keep_first, int pool, int64_t pooled_row_offset, int pool_here,
+                            int heads, int kv_heads, int maps, ca_maps mp, int dim, int vdim, int n_tok, int n_kv, float * scratch, size_t scratch_floats, float * out, int64_t out_stride, const int32_t * dyn_dev, void * stream);
 // the same kernel with the mask kind, pooled far blocks and a learned sink as parameters (`chunk` is the block's or the window's size)
 extern "C" int pi_op_window_attention(const float * q, int64_t q_stride, float * k_cache, float * v_cache, const int32_t * cell_pos_dev, const uint32_t * mask_dev, const int32_t * pos_dev,
                                       const float * head_bias_dev, const float * sink_dev, const float * gate_dev, int64_t gate_stride, int gate_act, float scale, float out_mult, int weights, float softcap, int mask_kind, int chunk,
                                       int pool, int64_t pooled_row_offset, int pool_here, int heads, int kv_heads, int dim, int vdim, int n_tok, int n_kv, float * scratch, size_t scratch_floats, float * out, int64_t out_stride,
                                       const int32_t * dyn_dev, void * stream) {
+    return window_attention(q, q_stride, k_cache, v_cache, cell_pos_dev, mask_dev, pos_dev, head_bias_dev, sink_dev, gate_dev, gate_stride, gate_act, scale, out_mult, weights, softcap, mask_kind, chunk, 0, pool, pooled_row_offset, pool_here,
+                            heads, kv_heads, 1, ca_maps{ 0.0f, 0.0f }, dim, vdim, n_tok, n_kv, scratch, scratch_floats, out, out_stride, dyn_dev, stream);
+}
+// soft-max over a window and the sequence's first keep_first positions; maps = 2: differential heads
+extern "C" int pi_op_diff_attention(const float * q, int64_t q_stride, const float * k_cache, const float * v_cache, const int32_t * cell_pos_dev, const uint32_t * mask_dev, const int32_t * pos_dev, float scale, int size, int keep_first,
+                                    int maps, float lam, float out_mult, float eps, int heads, int kv_heads, int dim, int vdim, int n_tok, int n_kv, float * scratch, size_t scratch_floats, float * out, int64_t out_stride,
+                                    const int32_t * dyn_dev, void * stream) {
+    return window_attention(q, q_stride, (float *) k_cache, (float *) v_cache, cell_pos_dev, mask_dev, pos_dev, nullptr, nullptr, nullptr, 0, PI_ACT_NONE, scale, out_mult, PI_WEIGHTS_SOFTMAX, 0.0f, PI_MASK_WINDOW, size, keep_first, 0, 0, 0,
+                            heads, kv_heads, maps, ca_maps{ lam, eps }, dim, vdim, n_tok, n_kv, scratch, scratch_floats, out, out_stride, dyn_dev, stream);
+}
+static int window_attention(const float * q, int64_t q_stride, float * k_cache, float * v_cache, const int32_t * cell_pos_dev, const uint32_t * mask_dev, const int32_t * pos_dev, const float * head_bias_dev, const float * sink_dev,
+                            const float * gate_dev, int64_t gate_stride, int gate_act, float scale, float out_mult, int weights, float softcap, int mask_kind, int chunk, int keep_first, int pool, int64_t pooled_row_offset, int pool_here,
+                            int heads, int kv_heads, int maps, ca_maps mp, int dim, int vdim, int n_tok, int n_kv, float * scratch, size_t scratch_floats, float * out, int64_t out_stride, const int32_t * dyn_dev, void * stream) {
     if (n_tok <= 0) return 0;
+    if (maps != 1 && maps != 2) { pi_set_error("pi_op_diff_attention: %d maps per head (1 or 2)", maps); return -1; }
+    if (maps == 2 && (head_bias_dev || sink_dev || gate_dev || weights != PI_WEIGHTS_SOFTMAX || pool_here || pool > 0)) { pi_set_error("pi_op_diff_attention: heads of two maps are a plain soft-max over the cells themselves"); return -1; }
+    if (keep_first < 0 || q_stride < (int64_t) heads * maps * dim) { pi_set_error("pi_op_diff_attention: %d kept positions, query rows of %lld floats for %d heads of %d x %d values", keep_first, (long long) q_stride, heads, maps, dim); return -1; }
     if (mask_kind != PI_MASK_CHUNK && mask_kind != PI_MASK_WINDOW) { pi_set_error("pi_op_window_attention: mask kind %d is unknown", mask_kind); return -1; }
     if (pool < 0 || (pool > 0 && (mask_kind != PI_MASK_WINDOW || chunk < 1 || pooled_row_offset < n_kv || pooled_row_offset > 0x3fffffff))) { pi_set_error("pi_op_window_attention: pooled blocks need a window and their rows behind the %d cells", n_kv); return -1; }
     if (sink_dev && weights == PI_WEIGHTS_SIGMOID) { pi_set_error("pi_op_window_attention: a sink belongs to a soft-max"); return -1; }
@@ -470,25 +549,29 @@ extern "C" int pi_op_window_attention(const float * q, int64_t q_stride, float *
     if (weights != PI_WEIGHTS_SIGMOID && weights != PI_WEIGHTS_SOFTMAX && weights != PI_WEIGHTS_SOFTMAX_SINK) { pi_set_error("pi_op_chunk_attention: weights of kind %d are unknown", weights); return -1; }
     if (heads < 1 || kv_heads < 1 || heads % kv_heads || dim < 1 || vdim < 1 || chunk < 0) { pi_set_error("pi_op_chunk_attention: %d query heads over %d key / value heads, sizes %d / %d, chunk %d", heads, kv_heads, dim, vdim, chunk); return -1; }
     int hpg = heads / kv_heads, splits = 1;                            // query heads of a key head that one workgroup serves: all of them, unless their outputs or the LDS plan say otherwise
-    while (hpg > 1 && (hpg * vdim > 256 * CA_MAXOUT || (size_t) hpg * dim * sizeof(float) > 24 * 1024)) { splits *= 2; hpg = (heads / kv_heads + splits - 1) / splits; }
+    while (hpg > 1 && (maps * hpg * vdim > 256 * CA_MAXOUT || (size_t) maps * hpg * dim * sizeof(float) > 24 * 1024)) { splits *= 2; hpg = (heads / kv_heads + splits - 1) / splits; }
     int tile = CA_TILE;
-    auto lds_of = [&](int tl) { return ((size_t) hpg * dim + (size_t) tl * std::max(dim + 1, vdim) + (size_t) tl * hpg + (size_t) 3 * hpg) * sizeof(float); };
+    auto lds_of = [&](int tl) { const size_t nr = (size_t) maps * hpg; return std::max(nr * dim + (size_t) tl * std::max(maps * dim + 1, vdim) + (size_t) tl * nr + 3 * nr, maps > 1 ? nr * vdim : (size_t) 0) * sizeof(float); };
     while (tile > 4 && lds_of(tile) > 60 * 1024) tile >>= 1;
     const size_t lds = std::max(lds_of(tile), pool_here ? (size_t) pool * sizeof(int) : (size_t) 0);
     const int n_z = (heads / kv_heads + hpg - 1) / hpg;
     // few tokens and a soft-max: the cell range is cut into splits that run side by side, merged by a second small launch (needs scratch for every split's share)
     int split_cells = 0, n_cs = weights != PI_WEIGHTS_SIGMOID && scratch ? ca_cell_splits(n_tok, kv_heads, n_z, n_kv, &split_cells) : 0;
-    if (n_cs < 2 || (size_t) n_tok * heads * n_cs * (vdim + 2) > scratch_floats) { n_cs = 1; split_cells = 0; }
-    if (hpg * vdim > 256 * CA_MAXOUT || lds > 60 * 1024) { pi_set_error("pi_op_chunk_attention: %d query heads per key head of sizes %d / %d are beyond the kernel (LDS %zu bytes)", hpg, dim, vdim, lds); return -1; }
+    if (n_cs < 2 || (size_t) n_tok * heads * maps * n_cs * (vdim + 2) > scratch_floats) { n_cs = 1; split_cells = 0; }
+    if (maps * hpg * vdim > 256 * CA_MAXOUT || lds > 60 * 1024) { pi_set_error("pi_op_chunk_attention: %d query heads per key head of sizes %d / %d are beyond the kernel (LDS %zu bytes)", hpg, dim, vdim, lds); return -1; }
     const int acct = pi_account_n_kv() > 0 ? pi_account_n_kv() : n_kv;
-    const double visible = chunk > 0 ? std::min(acct, chunk) + (pool > 0 ? std::max(acct - chunk, 0) / pool : 0) : acct;
-#define CA_GO(R)     PI_KT_LAUNCH(PI_KT_ATT, 0, std::min(n_tok, PI_KT_MAXNT - 1), 4.0 * visible * kv_heads * (dim + vdim) + 4.0 * n_tok * heads * (dim + vdim), k_chunk_attention<R>, dim3((unsigned) n_tok, (unsigned) kv_heads, (unsigned) (n_z * n_cs + (pool_here ? 1 : 0))), dim3(256), lds, \
+    const double visible = chunk > 0 ? std::min(acct, chunk) + (pool > 0 ? std::max(acct - chunk, 0) / pool : std::min(std::max(acct - chunk, 0), keep_first)) : acct;
+#define CA_GO(R, MP)     PI_KT_LAUNCH(PI_KT_ATT, 0, std::min(n_tok, PI_KT_MAXNT - 1), 4.0 * visible * kv_heads * (maps * dim + vdim) + 4.0 * n_tok * heads * (maps * dim + vdim), (k_chunk_attention<R, MP>), dim3((unsigned) n_tok, (unsigned) kv_heads, (unsigned) (n_z * n_cs + (pool_here ? 1 : 0))), dim3(256), lds, \
                  (hipStream_t) stream, q, q_stride, k_cache, v_cache, cell_pos_dev, mask_dev, pos_dev, head_bias_dev, gate_dev, gate_stride, gate_act, scale, out_mult, weights, softcap, chunk, heads, kv_heads, dim, vdim, n_kv, tile, hpg, out, out_stride, \
-                 dyn_dev, sink_dev, mask_kind, pool, (int) pooled_row_offset, pool_here ? n_z * n_cs : 0, n_z, n_cs, split_cells, scratch, pi_abort_word());
-    CA_GO(4);                                                          // (deeper rounds were measured for single tokens: no gain, the registers they take cost as much as the trips they save)
+                 dyn_dev, sink_dev, mask_kind, pool, (int) pooled_row_offset, pool_here ? n_z * n_cs : 0, n_z, n_cs, split_cells, scratch, keep_first, mp, pi_abort_word());
+    if (maps == 2) { CA_GO(4, 2); } else { CA_GO(4, 1); }              // (deeper rounds were measured for single tokens: no gain, the registers they take cost as much as the trips they save)
 #undef CA_GO
     PI_CHECK_LAUNCH();
-    if (split_cells > 0) {
+    if (split_cells > 0 && maps == 2) {
+        PI_KT_LAUNCH(PI_KT_ATT, 0, std::min(n_tok, PI_KT_MAXNT - 1), 4.0 * n_tok * heads * (2.0 * n_cs * (vdim + 2) + vdim), k_attention_combine_maps, dim3((unsigned) n_tok, (unsigned) heads), dim3(128), (size_t) 2 * vdim * sizeof(float),
+                     (hipStream_t) stream, scratch, n_cs, heads, vdim, mp, out_mult, out, out_stride, pi_abort_word());
+        PI_CHECK_LAUNCH();
+    } else if (split_cells > 0) {
         PI_KT_LAUNCH(PI_KT_ATT, 0, std::min(n_tok, PI_KT_MAXNT - 1), 4.0 * n_tok * heads * ((double) n_cs * (vdim + 2) + vdim), k_attention_combine, dim3((unsigned) n_tok, (unsigned) heads), dim3(128), 0, (hipStream_t) stream,
                      scratch, n_cs, heads, vdim, sink_dev, weights, gate_dev, gate_stride, gate_act, out_mult, out, out_stride, pi_abort_word());
         PI_CHECK_LAUNCH();

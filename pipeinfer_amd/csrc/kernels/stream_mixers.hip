@@ -2,6 +2,7 @@
 // with a rotated key part and a sliding window.  Everything here is fp32 in both precisions of the engine: streams, norms, gates and their running maximum, angles.
 //
 //   k_hyper_step       x_t <- sum_s mix[s][t] x_s + out[t] y over the streams of a token, the next sublayer's input sum_s in[s] x_s and its RMS norm in one pass over the row
+//                      (one stream: the plain pre-norm residual, x <- x + y [+ a fixed vector], and the norm of what reads it next)
 //   k_memory_gates     capped log gates and their running maximum (a max-plus scan over the tokens of a sequence), as factors the linear recurrence takes per token
 //   k_memory_norm      the memory's output divided by its normaliser, per-head RMS norm, weight, output gate
 //   k_window_mask      the pass's mask rows restricted to a window of positions
@@ -21,7 +22,8 @@ static __device__ __forceinline__ float sm_sigmoid(float v) { return 1.0f / (1.0
 // one workgroup per token; a thread owns NG groups of VEC neighbouring values of ALL streams, so the step may run in place and only the next input's squares are summed across threads
 template <int S, int VEC, int NG>
 __global__ void __launch_bounds__(1024) k_hyper_step(const float * xin, int64_t xts, int64_t xss, int ns, const float * __restrict__ y, int64_t ys, const float * __restrict__ mix, const float * __restrict__ outc,
-                                                     const float * __restrict__ in_next, const float * __restrict__ w, float eps, int n, float * xo, float * __restrict__ h, int64_t hs, const int32_t * __restrict__ abort_w) {
+                                                     const float * __restrict__ in_next, const float * __restrict__ shift, const float * __restrict__ w, float eps, int n, float * xo, float * __restrict__ h, int64_t hs,
+                                                     const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w)) return;
     __shared__ float red[16];
     const int t = blockIdx.x;
@@ -59,9 +61,13 @@ __global__ void __launch_bounds__(1024) k_hyper_step(const float * xin, int64_t 
                 }
             }
             if (y) {
-                const float o = outc[d];
+                const float o = outc ? outc[d] : 1.0f;
 #pragma unroll
                 for (int e = 0; e < VEC; e++) v[e] = fmaf(o, yv[e], v[e]);
+            }
+            if (shift) {
+#pragma unroll
+                for (int e = 0; e < VEC; e++) v[e] += shift[i + e];
             }
             if (xo) {
                 float * dst = xo + ((int64_t) t * ns + d) * n + i;
@@ -89,11 +95,11 @@ __global__ void __launch_bounds__(1024) k_hyper_step(const float * xin, int64_t 
         else dst[0] = u[g][0] * inv * w[i];
     }
 }
-extern "C" int pi_op_hyper_step(const float * x_in, int64_t token_stride, int64_t stream_stride, int streams, const float * y, int64_t y_stride, const float * mix_dev, const float * out_dev, const float * in_next_dev,
-                                const float * w_dev, float eps, int n, int n_tok, float * x_out, float * h_out, int64_t h_stride, void * stream) {
+static int hyper_step(const float * x_in, int64_t token_stride, int64_t stream_stride, int streams, const float * y, int64_t y_stride, const float * mix_dev, const float * out_dev, const float * in_next_dev,
+                      const float * shift_dev, const float * w_dev, float eps, int n, int n_tok, float * x_out, float * h_out, int64_t h_stride, void * stream) {
     if (n_tok <= 0 || n <= 0) return 0;
     if (streams < 1 || streams > PI_MAX_STREAMS || n > 16384) { pi_set_error("pi_op_hyper_step: %d streams of %d values (at most %d of 16384)", streams, n, PI_MAX_STREAMS); return -1; }
-    if (!x_in || !w_dev || !h_out || (y && !out_dev)) { pi_set_error("pi_op_hyper_step: the streams, the norm's weight, its output and the factors of a sublayer's result are required"); return -1; }
+    if (!x_in || !w_dev || !h_out) { pi_set_error("pi_op_hyper_step: the streams, the norm's weight and its output are required"); return -1; }
     if (x_out == x_in && (stream_stride != n || token_stride != (int64_t) streams * n)) { pi_set_error("pi_op_hyper_step: in place the streams lie as they are stored"); return -1; }
     auto al = [](const void * p, int64_t stride) { return !p || (((uintptr_t) p % 16) == 0 && stride % 4 == 0); };
     const bool vec = n % 4 == 0 && al(x_in, token_stride) && stream_stride % 4 == 0 && al(y, y_stride) && al(w_dev, 0) && al(x_out, 0) && al(h_out, h_stride);
@@ -101,13 +107,22 @@ extern "C" int pi_op_hyper_step(const float * x_in, int64_t token_stride, int64_
     const int threads = ng > 1 ? 1024 : (groups + 63) / 64 * 64;
     const double bytes = 4.0 * n * n_tok * ((stream_stride ? streams : 1) + (y ? 1 : 0) + (x_out ? streams : 0) + 1);
 #define HS_GO(S, V, G) PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, bytes, (k_hyper_step<S, V, G>), dim3((unsigned) n_tok), dim3((unsigned) threads), 0, (hipStream_t) stream, x_in, token_stride, stream_stride, streams, y, y_stride, mix_dev, \
-                                    out_dev, in_next_dev, w_dev, eps, n, x_out, h_out, h_stride, pi_abort_word())
+                                    out_dev, in_next_dev, shift_dev, w_dev, eps, n, x_out, h_out, h_stride, pi_abort_word())
 #define HS_S(V, G) do { if (streams == 1) HS_GO(1, V, G); else if (streams == 2) HS_GO(2, V, G); else if (streams == 3) HS_GO(3, V, G); else if (streams == 4) HS_GO(4, V, G); else if (streams <= 8) HS_GO(8, V, G); else HS_GO(16, V, G); } while (0)
     if (vec) { if (ng == 1) HS_S(4, 1); else HS_S(4, 4); }
     else { if (ng == 1) HS_S(1, 1); else if (ng == 4) HS_S(1, 4); else HS_S(1, 16); }
 #undef HS_S
 #undef HS_GO
     PI_CHECK_LAUNCH(); return 0;
+}
+extern "C" int pi_op_hyper_step(const float * x_in, int64_t token_stride, int64_t stream_stride, int streams, const float * y, int64_t y_stride, const float * mix_dev, const float * out_dev, const float * in_next_dev,
+                                const float * w_dev, float eps, int n, int n_tok, float * x_out, float * h_out, int64_t h_stride, void * stream) {
+    if (n_tok > 0 && n > 0 && y && !out_dev) { pi_set_error("pi_op_hyper_step: the factors of a sublayer's result are required"); return -1; }
+    return hyper_step(x_in, token_stride, stream_stride, streams, y, y_stride, mix_dev, out_dev, in_next_dev, nullptr, w_dev, eps, n, n_tok, x_out, h_out, h_stride, stream);
+}
+// the same kernel over ONE stream: x <- x + y + shift, h = R(x) * w
+extern "C" int pi_op_residual_norm(const float * x_in, const float * y, int64_t y_stride, const float * shift_dev, const float * w_dev, float eps, int n, int n_tok, float * x_out, float * h_out, int64_t h_stride, void * stream) {
+    return hyper_step(x_in, n, n, 1, y, y_stride, nullptr, nullptr, nullptr, shift_dev, w_dev, eps, n, n_tok, x_out, h_out, h_stride, stream);
 }
 
 // ---- gates of the matrix memory -----------------------------------------------------------------------------------------------------------------------
@@ -226,7 +241,7 @@ extern "C" int pi_op_window_mask(const uint32_t * mask_dev, const int32_t * pos_
 // ---- the two latents -----------------------------------------------------------------------------------------------------------------------------------
 // grid (token, 2): the query latent; the key / value latent and the rotated key part
 __global__ void __launch_bounds__(256) k_latent_prepare(const float * __restrict__ p, int64_t ps, int q_rank, const float * __restrict__ qw, int rank, const float * __restrict__ kw, int rot, const float2 * __restrict__ cs,
-                                                        int n_pos, float eps, const int32_t * __restrict__ pos, float * __restrict__ cq, int64_t cqs, float * __restrict__ cache, const int32_t * __restrict__ dyn,
+                                                        int n_pos, int pairing, float eps, const int32_t * __restrict__ pos, float * __restrict__ cq, int64_t cqs, float * __restrict__ cache, const int32_t * __restrict__ dyn,
                                                         const int32_t * __restrict__ abort_w) {
     if (pi_aborted(abort_w)) return;
     __shared__ float red[4];
@@ -245,19 +260,24 @@ __global__ void __launch_bounds__(256) k_latent_prepare(const float * __restrict
     if (is_q) return;
     const float2 * row = cs + (int64_t) min(pos[t], n_pos - 1) * (rot / 2);
     for (int i = tid; i < rot; i += 256) {
-        const float2 c = row[i >> 1];
-        const float own = src[rank + i], other = src[rank + (i ^ 1)];
-        dst[rank + i] = (i & 1) ? own * c.x + other * c.y : own * c.x - other * c.y;
+        const pi_turn u = pi_turn_of(i, rot / 2, pairing);
+        const float2 c = row[u.angle];
+        const float own = src[rank + i], other = src[rank + u.mate];
+        dst[rank + i] = u.lead ? own * c.x - other * c.y : own * c.x + other * c.y;
     }
 }
 extern "C" int pi_op_latent_prepare(const float * p, int64_t p_stride, int q_rank, const float * q_norm_w, int kv_rank, const float * kv_norm_w, int rot_dim, const void * rotary_table, float eps, const int32_t * pos_dev, int n_tok,
                                     float * q_latent, int64_t q_latent_stride, float * cache_dev, const int32_t * dyn_dev, void * stream) {
+    return pi_op_latent_prepare_ex(p, p_stride, q_rank, q_norm_w, kv_rank, kv_norm_w, rot_dim, rotary_table, PI_PAIR_NEIGHBOURS, eps, pos_dev, n_tok, q_latent, q_latent_stride, cache_dev, dyn_dev, stream);
+}
+extern "C" int pi_op_latent_prepare_ex(const float * p, int64_t p_stride, int q_rank, const float * q_norm_w, int kv_rank, const float * kv_norm_w, int rot_dim, const void * rotary_table, int pairing, float eps, const int32_t * pos_dev,
+                                       int n_tok, float * q_latent, int64_t q_latent_stride, float * cache_dev, const int32_t * dyn_dev, void * stream) {
     if (n_tok <= 0) return 0;
     const float2 * cs = nullptr; int n_pos = 0, half = 0;
     pi_rotary_table_view(rotary_table, &cs, &n_pos, &half);
-    if (q_rank < 1 || kv_rank < 1 || rot_dim < 0 || (rot_dim & 1) || (rot_dim > 0 && (!cs || half != rot_dim / 2 || !pos_dev))) { pi_set_error("pi_op_latent_prepare: latents of %d and %d values, %d rotated ones with a table over them", q_rank, kv_rank, rot_dim); return -1; }
+    if (q_rank < 1 || kv_rank < 1 || rot_dim < 0 || (rot_dim & 1) || (rot_dim > 0 && (!cs || half != rot_dim / 2 || !pos_dev)) || (pairing != PI_PAIR_HALVES && pairing != PI_PAIR_NEIGHBOURS)) { pi_set_error("pi_op_latent_prepare: latents of %d and %d values, %d rotated ones with a table over them", q_rank, kv_rank, rot_dim); return -1; }
     if (p_stride < (int64_t) q_rank + kv_rank + rot_dim || q_latent_stride < q_rank || !dyn_dev || !q_norm_w || !kv_norm_w) { pi_set_error("pi_op_latent_prepare: row strides below the sizes, or no norm weights / cell table"); return -1; }
-    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 8.0 * n_tok * (q_rank + kv_rank + rot_dim), k_latent_prepare, dim3((unsigned) n_tok, 2), dim3(256), 0, (hipStream_t) stream, p, p_stride, q_rank, q_norm_w, kv_rank, kv_norm_w, rot_dim, cs, n_pos, eps, pos_dev,
+    PI_KT_LAUNCH(PI_KT_OTHER, 0, 1, 8.0 * n_tok * (q_rank + kv_rank + rot_dim), k_latent_prepare, dim3((unsigned) n_tok, 2), dim3(256), 0, (hipStream_t) stream, p, p_stride, q_rank, q_norm_w, kv_rank, kv_norm_w, rot_dim, cs, n_pos, pairing, eps, pos_dev,
                  q_latent, q_latent_stride, cache_dev, dyn_dev, pi_abort_word());
     PI_CHECK_LAUNCH(); return 0;
 }

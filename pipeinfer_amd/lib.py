@@ -209,3 +209,9 @@ def _declare(lib):
     lib.pi_op_latent_prepare.argtypes = [vp, i64, i32, vp, i32, vp, i32, vp, f32, vp, i32, vp, i64, vp, vp, vp]
     lib.pi_op_latent_attention_rot.argtypes = [vp, i64, vp, vp, vp, vp, vp, vp, i64, i32, f32, i32, i32, i32, i32, i32, vp, vp, i32, i32, vp, sz, vp, i64, vp, vp]
     lib.pi_op_latent_attention_rot_scratch_floats.argtypes = [i32, i32, i32, i32, i32]; lib.pi_op_latent_attention_rot_scratch_floats.restype = sz
+    # plain pre-norm blocks, latent attention in other pairs with a gate per value, differential attention
+    lib.pi_op_residual_norm.argtypes = [vp, vp, i64, vp, vp, f32, i32, i32, vp, vp, i64, vp]
+    lib.pi_op_latent_prepare_ex.argtypes = [vp, i64, i32, vp, i32, vp, i32, vp, i32, f32, vp, i32, vp, i64, vp, vp, vp]
+    lib.pi_op_latent_attention_gated.argtypes = [vp, i64, vp, vp, vp, vp, vp, vp, i64, i32, i32, f32, i32, i32, i32, i32, i32, vp, i32, vp, i32, i32, vp, sz, vp, i64, vp, vp]
+    lib.pi_op_qkv_prepare_maps.argtypes = [vp, vp, vp, i64, i32, i32, i32, i32, i32, vp, i32, vp, i32, vp, i64, vp, vp, vp, vp, vp]
+    lib.pi_op_diff_attention.argtypes = [vp, i64, vp, vp, vp, vp, vp, f32, i32, i32, i32, f32, f32, f32, i32, i32, i32, i32, i32, i32, vp, sz, vp, i64, vp, vp]
