@@ -502,7 +502,13 @@ def main():
     ap.add_argument("--compare-streams", nargs="?", const="w1024,w2048,w4096", default=None, metavar="SIZES",
                     help="instead of the default workload: the same measurements for the Rerizen design (residual streams, matrix memories, windowed latent attention behind a query latent) beside the Fasovik "
                          "design at equal sizes; one JSON line per size")
+    ap.add_argument("--compare-diff", nargs="?", const="w1024,w2048,w4096", default=None, metavar="SIZES",
+                    help="instead of the default workload: the same measurements for the Letevik design (differential attention in windows with kept first tokens, latent attention with a sink and a gate per "
+                         "value) beside the Rerizen design at equal sizes; one JSON line per size")
     args = ap.parse_args()
+    if args.compare_diff:
+        from pipeinfer_amd.tools import hybrid_bench
+        return hybrid_bench.main_diff(args.compare_diff.split(","), args.cache)
     if args.compare_streams:
         from pipeinfer_amd.tools import hybrid_bench
         return hybrid_bench.main_streams(args.compare_streams.split(","), args.cache)

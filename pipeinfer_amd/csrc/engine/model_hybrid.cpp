@@ -210,7 +210,12 @@ static bool read_vikarax_config(const pi::json & cfg, pi_hparams & hp, std::stri
 // a pair embedding's table and multipliers, where the description has one
 static bool read_pair_embedding(const pi::json & cfg, pi_hparams & hp, std::string & what) {
     if (!cfg.at("embedding.bigram") || cfg.at("embedding.bigram")->is_null()) return true;
-    if (int_at(cfg, "embedding.bigram.buckets", hp.pair_buckets) && int_at(cfg, "embedding.bigram.mul_prev", hp.pair_mul_prev) && int_at(cfg, "embedding.bigram.mul_cur", hp.pair_mul_cur) && hp.pair_buckets > 0) return true;
+    double prev, cur;
+    auto whole = [](double d) { return d >= 0 && d == std::floor(d) && d <= 9007199254740992.0; };           // (integers a JSON number holds exactly)
+    if (int_at(cfg, "embedding.bigram.buckets", hp.pair_buckets) && hp.pair_buckets > 0 && num_at(cfg, "embedding.bigram.mul_prev", prev) && num_at(cfg, "embedding.bigram.mul_cur", cur) && whole(prev) && whole(cur)) {
+        hp.pair_mul_prev = (int) ((int64_t) prev % hp.pair_buckets); hp.pair_mul_cur = (int) ((int64_t) cur % hp.pair_buckets);      // (only the rest matters to the row: the products stay small)
+        return true;
+    }
     what = "embedding.bigram needs a positive 'buckets', 'mul_prev' and 'mul_cur'"; return false;
 }
 

@@ -994,21 +994,23 @@ __global__ void __launch_bounds__(256) k_latent_combine(const float * __restrict
     for (int vv = blockIdx.z * 16 + wave; vv < min(vdim, (int) blockIdx.z * 16 + 16); vv += 4) {
         const uint16_t * wv = wuv + ((int64_t) h * vdim + vv) * rank;
         float a[4] = { 0.0f, 0.0f, 0.0f, 0.0f };
+        const bool mine = lane < nt;                                   // lane tt writes token t0 + tt; its gate is on the way while the row is summed
+        float g = mine ? gsh[lane] : 1.0f;
+        if (gate && gate_width > 1 && mine) g = gate[(int64_t) (t0 + lane) * gs + (int64_t) h * vdim + vv];
 #pragma unroll 4
         for (int r = lane; r < rank; r += 64) {
             const float w = hy_widen(wv[r]);
 #pragma unroll
             for (int tt = 0; tt < 4; tt++) a[tt] = fmaf(w, ol[tt * rank + r], a[tt]);
         }
+        if (gate && gate_width > 1 && gate_act == PI_ACT_SIGMOID) g = 1.0f / (1.0f + expf(-g));
+        float v = 0.0f;
 #pragma unroll
         for (int tt = 0; tt < 4; tt++) {
-            const float v = pi_lanes_sum<64>(a[tt]);
-            if (lane == 0 && tt < nt) {
-                float g = gsh[tt];
-                if (gate && gate_width > 1) { g = gate[(int64_t) (t0 + tt) * gs + (int64_t) h * vdim + vv]; if (gate_act == PI_ACT_SIGMOID) g = 1.0f / (1.0f + expf(-g)); }
-                out[(int64_t) (t0 + tt) * os + (int64_t) h * vdim + vv] = v * g;
-            }
+            const float s = pi_lanes_sum<64>(a[tt]);
+            if (lane == tt) v = s;
         }
+        if (mine) out[(int64_t) (t0 + lane) * os + (int64_t) h * vdim + vv] = v * g;
     }
 }
 

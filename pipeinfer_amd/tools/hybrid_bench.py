@@ -13,7 +13,10 @@ closest model, which is Vikarax at the same width, depth, attention sizes and wi
 gated shared one, a repeated run's input matrix) beside the closest model, which is Vikarax at the same width, depth, attention and expert sizes.
 
 `bench.py --compare-streams [SIZE,...]`: the Rerizen design (four residual streams mixed around every sublayer; matrix memories, attention with a query temperature, latent attention in windows behind a
-query latent) beside the closest model, which is Fasovik at the same width, depth, head and latent sizes and with as many feed-forward parameters per token."""
+query latent) beside the closest model, which is Fasovik at the same width, depth, head and latent sizes and with as many feed-forward parameters per token.
+
+`bench.py --compare-diff [SIZE,...]`: the Letevik design (plain pre-norm blocks; latent attention with a sink and a gate per value, differential attention in windows with kept first tokens behind short
+convolutions, in turn; a repeated run's vector) beside the closest model, which is Rerizen at the same width, depth, head, latent and feed-forward sizes."""
 import ctypes as C
 import json
 import os
@@ -254,6 +257,31 @@ def write_rerizen(folder, size, seed=1, streams=4):
     return write_random_tensors(folder, cfg, shapes, ones=("norm", "norm1", "norm2", ".in", ".out"), seed=seed)
 
 
+def write_letevik(folder, size, seed=1):
+    """layers in turn: latent attention, then differential attention (two maps of half the head size, so that its projections are those of the other designs' heads); window = the Vikarax model's chunk of
+    this size; layers 1 .. 2 are a (once-run) repeated run, so the run's vector is part of a pass"""
+    width, n_layer, heads, dim, vdim, rank, _, _, _, _, vocab = SIZES[size]
+    kv_heads, window, ff, rot, q_rank = VIKARAX[size][0], VIKARAX[size][2], rerizen_ff(size), dim // 2, width // 2
+    layers, shapes = [], {"embed": (vocab, width), "bigram": (65537, width), "loop.step": (1, width), "final.norm": (width,)}
+    for i in range(n_layer):
+        p, q, hd, hv = "l%d." % i, "l%d.mix." % i, heads * dim, heads * vdim
+        if i % 2:
+            mx = {"heads": heads, "kv_heads": kv_heads, "dim": dim // 2, "vdim": vdim, "scale": (dim // 2) ** -0.5, "diff": 0.4, "conv": 4, "rot": {"dims": dim // 2, "base": 10000.0}, "mask": {"size": window, "keep_first": 4}}
+            for n, rows in (("q", hd), ("k", kv_heads * dim), ("v", kv_heads * vdim)):
+                shapes.update({q + n: (rows, width), q + n + ".conv": (rows, 4)})
+            shapes.update({q + n: (dim // 2,) for n in ("lq1", "lk1", "lq2", "lk2")})
+        else:
+            mx = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "q_rank": q_rank, "kv_rank": rank, "scale": (dim + rot) ** -0.5, "rot": {"dims": rot, "base": 10000.0}}
+            shapes.update({q + "dq": (q_rank, width), q + "dq.norm": (q_rank,), q + "uq": (heads * (dim + rot), q_rank), q + "dkv": (rank + rot, width), q + "dkv.norm": (rank,), q + "uk": (hd, rank),
+                           q + "uv": (hv, rank), q + "sink": (heads,), q + "g": (hv, width)})
+        shapes[q + "o"] = (width, hv)
+        layers.append({"type": "attention" if i % 2 else "latent_attention", "mixer": mx, "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}})
+        shapes.update({p + "norm1": (width,), p + "norm2": (width,), p + "mlp.gate": (ff, width), p + "mlp.up": (ff, width), p + "mlp.down": (width, ff)})
+    cfg = {"architecture": "Letevik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"bigram": {"buckets": 65536, "mul_prev": 8191, "mul_cur": 31}},
+           "loop": {"start": 1, "stop": min(3, n_layer), "times": 1}, "layers": layers}
+    return write_random_tensors(folder, cfg, shapes, ones=("norm", "norm1", "norm2"), seed=seed)
+
+
 class KtRow(C.Structure):          # struct pi_kt_row (include/pipeinfer_ops.h)
     _fields_ = [("family", C.c_int32), ("type", C.c_int32), ("n_tok", C.c_int32), ("sampled_dropped", C.c_int32), ("shape_bytes", C.c_uint64), ("launches", C.c_uint64),
                 ("bytes_total", C.c_double), ("sampled", C.c_uint64), ("avg_us", C.c_double), ("avg_sampled_bytes", C.c_double)]
@@ -408,6 +436,26 @@ def main_streams(sizes, cache, n_prompt=512, n_decode=64):
     return 0
 
 
+def main_diff(sizes, cache, n_prompt=512, n_decode=64):
+    """Letevik beside Rerizen at equal sizes; one JSON line per size"""
+    lib = L.load()
+    L.check(lib.pi_device_init(0), "pi_device_init")
+    for size in sizes:
+        width, n_layer, heads, dim, vdim, rank, _, _, _, _, vocab = SIZES[size]
+        lev, rer = os.path.join(cache, "letevik-" + size), os.path.join(cache, "rerizen-" + size)
+        if not os.path.exists(os.path.join(lev, "model.safetensors")):
+            write_letevik(lev, size)
+        if not os.path.exists(os.path.join(rer, "model.safetensors")):
+            write_rerizen(rer, size)
+        out = {"size": size, "config": {"width": width, "layers": n_layer, "heads": heads, "kv_heads": VIKARAX[size][0], "dim": dim, "map_dim": dim // 2, "vdim": vdim, "rot_dim": dim // 2, "q_rank": width // 2,
+                                       "kv_rank": rank, "window": VIKARAX[size][2], "keep_first": 4, "conv": 4, "ff": rerizen_ff(size), "vocab": vocab, "n_prompt": n_prompt, "n_decode": n_decode, "rerizen": {"streams": 4}},
+               "letevik_bf16": measure(lib, lev, n_prompt, n_decode, True),
+               "rerizen_bf16": measure(lib, rer, n_prompt, n_decode, True), "data": "synthetic", "hbm_peak": HBM_PEAK}
+        print(json.dumps(out))
+        sys.stdout.flush()
+    return 0
+
+
 def main(sizes, cache, n_prompt=512, n_decode=64):
     lib = L.load()
     L.check(lib.pi_device_init(0), "pi_device_init")
@@ -436,7 +484,7 @@ def run_phase(design, size, phase, cache, n_prompt=512, n_decode=64):
     L.check(lib.pi_device_init(0), "pi_device_init")
     folder = os.path.join(cache, "%s-%s" % (design, size))
     if not os.path.exists(os.path.join(folder, "model.safetensors")):
-        {"vikarax": write_vikarax, "fasovik": write_fasovik, "rafusun": write_rafusun, "rarevik": write_rarevik, "rerizen": write_rerizen}[design](folder, size)
+        {"vikarax": write_vikarax, "fasovik": write_fasovik, "rafusun": write_rafusun, "rarevik": write_rarevik, "rerizen": write_rerizen, "letevik": write_letevik}[design](folder, size)
     model = LL.Model(folder)
     ctx = LL.Context(model, n_ctx=n_prompt + n_decode + 64, n_batch=n_prompt)
     ctx.set_precision(False)
@@ -457,7 +505,7 @@ def run_phase(design, size, phase, cache, n_prompt=512, n_decode=64):
 if __name__ == "__main__":
     import argparse
     ap = argparse.ArgumentParser(description="one phase of one folder-described design at one size (for `rocprofv3 --kernel-trace --stats -- python3 -m pipeinfer_amd.tools.hybrid_bench ...`)")
-    ap.add_argument("--design", choices=["vikarax", "fasovik", "rafusun", "rarevik", "rerizen"], required=True)
+    ap.add_argument("--design", choices=["vikarax", "fasovik", "rafusun", "rarevik", "rerizen", "letevik"], required=True)
     ap.add_argument("--size", choices=sorted(SIZES), default="w2048")
     ap.add_argument("--phase", choices=["prefill", "decode"], required=True)
     ap.add_argument("--cache", default=os.environ.get("PIPEINFER_CACHE", "/tmp/pipeinfer_models"))
